@@ -1,0 +1,102 @@
+/*
+ * trimkv_hybrid.h -- C ABI of libtrimkv_hybrid.so: the kernels of decoders that mix windowed attention with recurrent
+ * layers and routed experts, on MI355X (gfx950).
+ *
+ * Conventions as in trimkv_hip.h: device pointers throughout, work enqueued on `stream`, no allocation and no host
+ * synchronisation, 0 / negative trimkv_status / positive hipError_t, text of the last error of the calling thread from
+ * trimkv_hybrid_last_error().  `dtype` is the type of activations and matrices: TRIMKV_BF16 or TRIMKV_F32 (everything in
+ * true fp32).  Norm weights, biases, gates, router logits, recurrent state and the residual stream are fp32 always.
+ *
+ * Batches are packed: the tokens of all sequences of a step lie one after the other, sequence b owns tokens
+ * cu[b] .. cu[b+1]-1 (cu [batch+1] int32).  What a sequence leaves behind lives in a slot, slots[b] (int32); seen [slots][2]
+ * int32 holds the tokens and the steps a slot has seen before this step (trimkv_advance moves both on at its end).  Slot
+ * contents of a slot with 0 tokens are never read.
+ */
+#ifndef TRIMKV_HYBRID_H
+#define TRIMKV_HYBRID_H
+
+#include "trimkv_hip.h"
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+const char* trimkv_hybrid_last_error(void);
+
+/* x[t] = table[ids[t]] * scale as fp32 rows of x_stride elements (zeros behind `width`); xh (optional): the same in dtype.
+ * Ids outside [0, vocab) are clamped. */
+int trimkv_embed_scaled(const int64_t* ids, const void* table, float scale, float* x, void* xh, int tokens, int vocab, int width,
+                        int x_stride, int dtype, void* stream);
+
+/* out[t][o] = sum_k x[t][k] w[o][k], fp32 x and out, fp32 products and sums (bf16 w on the matrix cores: x split exactly into
+ * three bf16 terms).  k and x_stride multiples of 4, w_stride a multiple of 8; 16-byte aligned. */
+int trimkv_linear_f32(const float* x, int64_t x_stride, const void* w, int64_t w_stride, float* out, int rows, int n, int k, int dtype, void* stream);
+
+/* x[t] += w * y' / sqrt(mean(y'^2) + eps), y' = y[t] or, with y_weight [tokens][top], sum_j y_weight[t][j] * y[t * top + j].
+ * xh (optional): the new x in dtype, same stride. width <= 16384. */
+int trimkv_residual_norm(const void* y, int64_t y_stride, const float* y_weight, int top, float* x, const float* w, void* xh,
+                         int tokens, int width, int x_stride, float eps, int dtype, void* stream);
+
+/* out[i] = w * x[r] / sqrt(mean(x[r]^2) + eps) with r = rows[i] (NULL: r = i); out [count][width] in dtype. */
+int trimkv_rms_rows(const float* x, int x_stride, const int64_t* rows, const float* w, void* out, int count, int width, float eps, int dtype, void* stream);
+
+/* RMS norm of q over all its heads at once, likewise k (weights of those sizes); v is copied.  proj rows hold q, k, v at
+ * element offsets q_off, k_off, v_off.  Outputs [tokens][heads][dim_stride] / [tokens][kv_heads][(v)dim_stride], zeros behind
+ * dim / vdim.  With slots and seen (one token per sequence): k and v are the window rings and the token goes into its slot. */
+int trimkv_qkv_norm(const void* proj, int64_t proj_stride, int q_off, int k_off, int v_off, const float* q_weight, const float* k_weight, float eps,
+                    int heads, int kv_heads, int dim, int vdim, int dim_stride, int vdim_stride, void* q, void* k, void* v,
+                    const int32_t* slots, const int32_t* seen, int keep_first, int window, int tokens, int dtype, void* stream);
+
+/* Window rings [slot][kv_heads][keep_first + window][dim_stride]: position p < keep_first owns row p, a later one row
+ * keep_first + (p - keep_first) % window.  Stores those tokens of a portion that no later token of it overwrites. */
+int trimkv_ring_store(const void* k, const void* v, const int32_t* cu, const int32_t* slots, const int32_t* seen, void* ring_k, void* ring_v,
+                      int batch, int max_len, int kv_heads, int dim_stride, int vdim_stride, int keep_first, int window, int dtype, void* stream);
+
+/* Attention of portions: position i sees j <= i with i - j < window or j < keep_first; earlier tokens from the rings (which
+ * must not hold this portion yet), the portion's own from k and v.  out [tokens][heads * vdim] = attention * sigmoid(gate),
+ * gate rows gate_stride apart. Padded sizes are multiples of 8 up to 512. */
+int trimkv_window_prefill(const void* q, const void* k, const void* v, const void* ring_k, const void* ring_v, const int32_t* cu,
+                          const int32_t* slots, const int32_t* seen, const void* gate, int64_t gate_stride, void* out, int batch, int max_len,
+                          int heads, int kv_heads, int dim, int vdim, int dim_stride, int vdim_stride, int keep_first, int window,
+                          float scale, int dtype, void* stream);
+
+/* Attention of one new token per sequence, already stored in the rings (seen does not count it yet).  splits > 1: rows of a
+ * sequence are split over that many workgroups, workspace [batch][heads][splits][vdim + 2] floats. */
+int trimkv_window_decode_splits(int batch, int kv_heads, int capacity);
+int trimkv_window_decode(const void* q, const void* ring_k, const void* ring_v, const int32_t* slots, const int32_t* seen,
+                         const void* gate, int64_t gate_stride, void* out, int batch, int heads, int kv_heads, int dim, int vdim,
+                         int dim_stride, int vdim_stride, int keep_first, int window, float scale, int splits, float* workspace,
+                         int dtype, void* stream);
+
+/* mLSTM over portions (equations in csrc/mlstm.hip). gates [tokens][2 heads]: W_i h, W_f h without biases.  state
+ * [slot][heads][dim][vdim]; norm_state [2][num_slots][heads][dim + 1] (n and m, by parity of the slot's steps).
+ * out [tokens][heads][vdim] fp32, before the head norm.  dim up to 512. */
+int trimkv_mlstm(const void* proj, int64_t proj_stride, int q_off, int k_off, int v_off, const float* gates, const float* i_bias,
+                 const float* f_bias, float gate_cap, float* state, float* norm_state, const int32_t* cu, const int32_t* slots, const int32_t* seen,
+                 float* out, int batch, int max_len, int heads, int dim, int vdim, int num_slots, float q_scale, int dtype, void* stream);
+
+/* out[t][h][:] = w[h] * o / sqrt(mean(o^2) + eps) * sigmoid(gate), o [tokens][heads][vdim] fp32. */
+int trimkv_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int tokens, int heads, int vdim, float eps, int dtype, void* stream);
+
+/* seen[slots[b]] += {cu[b+1] - cu[b], 1}. */
+int trimkv_advance(int32_t* seen, const int32_t* slots, const int32_t* cu, int batch, void* stream);
+
+/* Sigmoid routing: choice = sigmoid(logits) + correction; `keep_groups` of `groups` equal groups of neighbours with the
+ * largest sums of their two largest choices are open; the `top` largest open choices win (lower index first among equals).
+ * weights: the plain sigmoids of the chosen. experts <= 1024. */
+int trimkv_moe_route(const float* logits, const float* correction, int32_t* ids, float* weights, int tokens, int experts, int top, int groups,
+                     int keep_groups, void* stream);
+
+/* Orders rows = tokens * top by expert: order [rows], offsets [experts + 1], tiles [1 + 2 * most]: their number, then
+ * (expert, first row) of every run of up to `tile` rows; most = rows < experts ? rows : (rows - experts) / tile + experts. */
+int trimkv_moe_plan(const int32_t* ids, int rows, int experts, int tile, int32_t* order, int32_t* offsets, int32_t* tiles, void* stream);
+
+/* One product per expert: w [experts][n_padded][k_padded], zeros in the padding (multiples of 64).  up: y[i] =
+ * relu(w x[order[i] / top])^2; else y[order[i]] = w x[i].  `tile` as in the plan: 16 or (bf16) 128. */
+int trimkv_moe_gemm(const void* x, int64_t x_stride, const void* w, void* y, int64_t y_stride, const int32_t* order, const int32_t* offsets,
+                    const int32_t* tiles, int rows, int experts, int tile, int top, int n, int n_padded, int k_padded, int up, int dtype, void* stream);
+
+#ifdef __cplusplus
+}
+#endif
+#endif

@@ -10,6 +10,7 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libtrimkv_hip.so")
+HYBRID_LIB_PATH = os.path.join(_HERE, "libtrimkv_hybrid.so")
 
 F32, BF16, F16 = 0, 1, 2
 SCORE_ALPHA, SCORE_KNORM_ALPHA = 0, 1
@@ -81,7 +82,28 @@ SIGNATURES = {
     "trimkv_stream_probe": (_i, [_p, _p, _i64, _i, _p, _p]),
 }
 
+# the same for trimkv_hybrid.h
+HYBRID_SIGNATURES = {
+    "trimkv_hybrid_last_error": (C.c_char_p, []),
+    "trimkv_embed_scaled": (_i, [_p, _p, _f, _p, _p, _i, _i, _i, _i, _i, _p]),
+    "trimkv_linear_f32": (_i, [_p, _i64, _p, _i64, _p, _i, _i, _i, _i, _p]),
+    "trimkv_residual_norm": (_i, [_p, _i64, _p, _i, _p, _p, _p, _i, _i, _i, _f, _i, _p]),
+    "trimkv_rms_rows": (_i, [_p, _i, _p, _p, _p, _i, _i, _f, _i, _p]),
+    "trimkv_qkv_norm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _f, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _p]),
+    "trimkv_ring_store": (_i, [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
+    "trimkv_window_prefill": (_i, [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
+    "trimkv_window_decode_splits": (_i, [_i, _i, _i]),
+    "trimkv_window_decode": (_i, [_p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p, _i, _p]),
+    "trimkv_mlstm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _f, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
+    "trimkv_head_norm_gate": (_i, [_p, _p, _i64, _p, _p, _i, _i, _i, _f, _i, _p]),
+    "trimkv_advance": (_i, [_p, _p, _p, _i, _p]),
+    "trimkv_moe_route": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _i, _p]),
+    "trimkv_moe_plan": (_i, [_p, _i, _i, _i, _p, _p, _p, _p]),
+    "trimkv_moe_gemm": (_i, [_p, _i64, _p, _p, _i64, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
+}
+
 _lib = None
+_hybrid = None
 
 
 def load():
@@ -100,6 +122,30 @@ def load():
         fn.argtypes = args
     _lib = lib
     return lib
+
+
+def load_hybrid():
+    """The ctypes handle of libtrimkv_hybrid.so (loaded once); raises if the library has not been built."""
+    global _hybrid
+    if _hybrid is not None:
+        return _hybrid
+    if not os.path.exists(HYBRID_LIB_PATH):
+        raise TrimKVLibraryError(
+            f"{HYBRID_LIB_PATH} is missing: build it with `python -m trimkv_amd.build hybrid` (hipcc, gfx950). "
+            "There is no CPU fallback.")
+    lib = C.CDLL(HYBRID_LIB_PATH)
+    for name, (res, args) in HYBRID_SIGNATURES.items():
+        fn = getattr(lib, name)
+        fn.restype = res
+        fn.argtypes = args
+    _hybrid = lib
+    return lib
+
+
+def check_hybrid(rc: int, what: str) -> None:
+    if rc != 0:
+        msg = load_hybrid().trimkv_hybrid_last_error().decode("utf-8", "replace")
+        raise TrimKVLibraryError(f"{what} failed with status {rc}: {msg}")
 
 
 def check(rc: int, what: str) -> None:

@@ -1,7 +1,8 @@
-"""Build libtrimkv_hip.so (the C-ABI library of HIP kernels) in-tree for gfx950.
+"""Build the C-ABI libraries of HIP kernels in-tree for gfx950: libtrimkv_hip.so (the TRIM-KV cache path and its decoders)
+and libtrimkv_hybrid.so (decoders with windowed attention, recurrent layers and routed experts).
 
-Usage: ``python -m trimkv_amd.build [--changed]`` (hipcc cross-compiles without a GPU; ``--changed`` recompiles only
-the sources whose object file is older than its inputs).
+Usage: ``python -m trimkv_amd.build [--changed] [hip|hybrid ...]`` (hipcc cross-compiles without a GPU; ``--changed``
+recompiles only the sources whose object file is older than its inputs; no name: both libraries).
 """
 from __future__ import annotations
 
@@ -14,7 +15,10 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 INCLUDE = os.path.join(os.path.dirname(HERE), "include")
 LIB_PATH = os.path.join(HERE, "libtrimkv_hip.so")
+HYBRID_LIB_PATH = os.path.join(HERE, "libtrimkv_hybrid.so")
 SOURCES = ["api.hip", "append.hip", "evict.hip", "attn_decode.hip", "attn_decode_append.hip", "attn_decode_pieces.hip", "attn_decode_append_pieces.hip", "attn_decode_append_gated.hip", "attn_decode_append_pieces_gated.hip", "pieces_plan.hip", "attn_prefill.hip", "gate.hip", "stream_probe.hip", "decoder_ops.hip"]
+HYBRID_SOURCES = ["hybrid_ops.hip", "window_attn.hip", "mlstm.hip", "moe.hip"]
+LIBRARIES = {"hip": (LIB_PATH, SOURCES), "hybrid": (HYBRID_LIB_PATH, HYBRID_SOURCES)}
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-I" + INCLUDE, "-I" + CSRC,
@@ -41,33 +45,36 @@ def _stale(src: str, obj: str) -> bool:
     return any(os.path.getmtime(d) > os.path.getmtime(obj) for d in deps)
 
 
-def build(verbose: bool = True, only_changed: bool = False) -> str:
-    """Compile every source (or, with ``only_changed``, the ones whose object is older than its inputs) and link."""
+def build(verbose: bool = True, only_changed: bool = False, libraries=("hip", "hybrid")) -> str:
+    """Compile every source of the named libraries (or, with ``only_changed``, the ones whose object is older than its
+    inputs) and link them."""
     hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
     objdir = os.path.join(HERE, "build")
     os.makedirs(objdir, exist_ok=True)
-    srcs = [s for s in SOURCES if os.path.exists(os.path.join(CSRC, s))]
-    objs = [os.path.join(objdir, s.replace(".hip", ".o")) for s in srcs]
-    all_objs = objs
+    obj_of = lambda s: os.path.join(objdir, s.replace(".hip", ".o"))
+    srcs = [s for name in libraries for s in LIBRARIES[name][1]]
     if only_changed:
-        keep = [i for i, (s, o) in enumerate(zip(srcs, objs)) if _stale(s, o)]
-        srcs, objs = [srcs[i] for i in keep], [objs[i] for i in keep]
+        srcs = [s for s in srcs if _stale(s, obj_of(s))]
 
-    def compile_one(pair):
-        src, obj = pair
-        return _run([hipcc] + HIPCC_FLAGS + ["-c", os.path.join(CSRC, src), "-o", obj])
+    def compile_one(src):
+        return _run([hipcc] + HIPCC_FLAGS + ["-c", os.path.join(CSRC, src), "-o", obj_of(src)])
 
     if srcs:
         with ThreadPoolExecutor(max_workers=min(os.cpu_count() or 4, 8, len(srcs))) as ex:
-            for src, out in zip(srcs, ex.map(compile_one, zip(srcs, objs))):
+            for src, out in zip(srcs, ex.map(compile_one, srcs)):
                 if verbose and out.strip():
                     print("[%s]\n%s" % (src, out))
-    _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_PATH] + all_objs)
-    if verbose:
-        print("built", LIB_PATH)
-    return LIB_PATH
+    for name in libraries:
+        path, sources = LIBRARIES[name]
+        part = "%s.%d" % (path, os.getpid())       # linked beside and renamed: nobody loads half a library
+        _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", part] + [obj_of(s) for s in sources])
+        os.replace(part, path)
+        if verbose:
+            print("built", path)
+    return LIBRARIES[libraries[-1]][0]
 
 
 if __name__ == "__main__":
-    build(only_changed="--changed" in sys.argv[1:])
+    names = [a for a in sys.argv[1:] if not a.startswith("--")]
+    build(only_changed="--changed" in sys.argv[1:], libraries=tuple(names) or ("hip", "hybrid"))
     sys.exit(0)

@@ -1,0 +1,354 @@
+// The row-wise work of the hybrid decoders, one launch each; the residual stream is fp32.
+//
+//   trimkv_embed_scaled    x = table[id] * scale
+//   trimkv_linear_f32      fp32 rows times a narrow matrix with fp32 results (routers, gates of a recurrence)
+//   trimkv_residual_norm   x += w * rms(y), y one row or a weighted sum of several (the experts of a token)
+//   trimkv_rms_rows        w * rms(x) of chosen rows
+//   trimkv_qkv_norm        RMS norm over the whole q and the whole k projection; q, k, v into head-major padded rows, or k
+//                          and v straight into the window ring (decode)
+//   trimkv_ring_store      the rows of a prompt that outlive it, into the window ring
+//   trimkv_head_norm_gate  per-head RMS norm, weight and sigmoid gate behind a recurrence
+//   trimkv_advance         tokens and steps seen per sequence slot
+#include "hybrid.hip.h"
+
+namespace trimkv {
+
+// ---- embedding -------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void embed_kernel(const int64_t* ids, const T* table, float scale, float* x, T* xh, int vocab, int width, int xs) {
+    const int64_t t = blockIdx.x;
+    const int64_t id = min(max(ids[t], (int64_t)0), (int64_t)vocab - 1);
+    for (int i = threadIdx.x; i < xs; i += 256) {
+        const float f = i < width ? ld(table + id * width + i) * scale : 0.0f;
+        x[t * xs + i] = f;
+        if (xh) st(xh + t * xs + i, f);
+    }
+}
+
+// ---- fp32 rows times a narrow matrix ---------------------------------------------------------
+// General form: one wavefront per (row, output).
+template <typename T>
+__global__ __launch_bounds__(256) void linear_f32_kernel(const float* x, int64_t xs, const T* w, int64_t ws, float* out, int64_t units, int n, int k) {
+    const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (unit >= units) return;
+    const int64_t t = unit / n;
+    const int o = (int)(unit - t * n), lane = threadIdx.x & 63;
+    const float* xr = x + t * xs;
+    const T* wr = w + o * ws;
+    float acc = 0.0f;
+    for (int i = lane * 4; i < k; i += 256) {
+        const float4 a = ld4(xr + i), b = ld4(wr + i);
+        acc += a.x * b.x + a.y * b.y + a.z * b.z + a.w * b.w;
+    }
+    acc = wave_sum_f(acc);
+    if (lane == 0) out[unit] = acc;
+}
+
+// bf16 weights on the matrix cores: a row's fp32 values are split exactly into three bf16 terms, so every product is an
+// fp32 product.  A workgroup owns 16 rows and 16 * NT outputs; its WAVES wavefronts split k and meet in LDS.
+// Operands straight from memory: lane l holds 8 consecutive k of row (or output) l % 16 at k-group l / 16.
+template <int NT, int WAVES>
+__global__ __launch_bounds__(WAVES * 64) void linear_f32_mfma_kernel(const float* x, int64_t xs, const bf16_t* w, int64_t ws, float* out, int rows, int n, int k) {
+    __shared__ float part[WAVES][NT][256];
+    const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, r = lane & 15, kg = lane >> 4;
+    const int row0 = blockIdx.x * 16, n0 = blockIdx.y * 16 * NT;
+    const float* xr = x + (int64_t)min(row0 + r, rows - 1) * xs;
+    const bf16_t* wr[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) wr[j] = w + (int64_t)min(n0 + 16 * j + r, n - 1) * ws;
+    hy_f32x4 acc[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[j] = {0.f, 0.f, 0.f, 0.f};
+    for (int i = wv * 32; i < k; i += WAVES * 32) {     // k is a multiple of 32
+        const float4 a = *(const float4*)(xr + i + kg * 8), b = *(const float4*)(xr + i + kg * 8 + 4);
+        hy_bf16x8 wf[NT];
+#pragma unroll
+        for (int j = 0; j < NT; ++j) wf[j] = *(const hy_bf16x8*)(wr[j] + i + kg * 8);
+        uint32_t s0[3], s1[3], s2[3], s3[3];
+        split2<3>(a.x, a.y, s0); split2<3>(a.z, a.w, s1); split2<3>(b.x, b.y, s2); split2<3>(b.z, b.w, s3);
+#pragma unroll
+        for (int e = 2; e >= 0; --e) {
+            const hy_bf16x8 xf = __builtin_bit_cast(hy_bf16x8, (hy_u32x4){s0[e], s1[e], s2[e], s3[e]});
+#pragma unroll
+            for (int j = 0; j < NT; ++j) acc[j] = mfma16(xf, wf[j], acc[j]);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j) *(hy_f32x4*)&part[wv][j][lane * 4] = acc[j];
+    __syncthreads();
+    for (int e = tid; e < NT * 256; e += WAVES * 64) {
+        const int j = e >> 8, idx = e & 255;
+        float s = 0.0f;
+#pragma unroll
+        for (int v = 0; v < WAVES; ++v) s += part[v][j][idx];
+        const int l = idx >> 2, row = row0 + 4 * (l >> 4) + (idx & 3), col = n0 + 16 * j + (l & 15);
+        if (row < rows && col < n) out[(int64_t)row * n + col] = s;
+    }
+}
+
+// ---- residual += w * rms(y) --------------------------------------------------------------------
+struct ResidualNormArgs {
+    const void* y; int64_t y_stride; const float* y_weight; int top;
+    float* x; const float* w; void* xh; int width, xs; float eps;
+};
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) {
+    extern __shared__ float row[];     // width floats: y of this token, summed over its experts
+    __shared__ float part[4];
+    const int64_t t = blockIdx.x;
+    const int tid = threadIdx.x;
+    const T* y = (const T*)a.y + t * a.top * a.y_stride;
+    float ss = 0.0f;
+    if constexpr (VEC) {
+        for (int i = tid * 4; i < a.width; i += 1024) {
+            float4 s;
+            if (a.y_weight) {
+                s = make_float4(0.f, 0.f, 0.f, 0.f);
+                for (int j = 0; j < a.top; ++j) {
+                    const float wt = a.y_weight[t * a.top + j];
+                    const float4 f = ld4(y + j * a.y_stride + i);
+                    s.x += wt * f.x; s.y += wt * f.y; s.z += wt * f.z; s.w += wt * f.w;
+                }
+            } else s = ld4(y + i);
+            *(float4*)(row + i) = s;
+            ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
+        }
+    } else {
+        for (int i = tid; i < a.width; i += 256) {
+            float s = 0.0f;
+            if (a.y_weight) for (int j = 0; j < a.top; ++j) s += a.y_weight[t * a.top + j] * ld(y + j * a.y_stride + i);
+            else s = ld(y + i);
+            row[i] = s;
+            ss += s * s;
+        }
+    }
+    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+    float* xr = a.x + t * a.xs;
+    T* hr = (T*)a.xh + t * a.xs;
+    if constexpr (VEC) {
+        for (int i = tid * 4; i < a.width; i += 1024) {     // a thread re-reads what it wrote itself
+            const float4 s = *(const float4*)(row + i), w = *(const float4*)(a.w + i);
+            float4 f = *(const float4*)(xr + i);
+            f.x += s.x * inv * w.x; f.y += s.y * inv * w.y; f.z += s.z * inv * w.z; f.w += s.w * inv * w.w;
+            *(float4*)(xr + i) = f;
+            if (a.xh) st4(hr + i, f);
+        }
+    } else {
+        for (int i = tid; i < a.width; i += 256) {
+            const float f = xr[i] + row[i] * inv * a.w[i];
+            xr[i] = f;
+            if (a.xh) st(hr + i, f);
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void rms_rows_kernel(const float* x, int xs, const int64_t* rows, const float* w, T* out, int width, float eps) {
+    __shared__ float part[4];
+    const int64_t t = blockIdx.x;
+    const float* xr = x + (rows ? rows[t] : t) * xs;
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < width; i += 256) ss += xr[i] * xr[i];
+    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)width + eps);
+    for (int i = threadIdx.x; i < width; i += 256) st(out + t * width + i, xr[i] * inv * w[i]);
+}
+
+// ---- q and k normed over all their heads ---------------------------------------------------------
+struct QkvNormArgs {
+    const void* p; int64_t p_stride; int q_off, k_off, v_off;
+    const float* qw; const float* kw; float eps;
+    int H, G, D, Dv, Dp, Dvp;
+    void* q; void* k; void* v;                       // [T][heads][padded dim]
+    const int32_t* slots; const int32_t* seen;       // both given: k and v rows go into the rings k, v [slot][G][cap][padded dim]
+    int keep, size;
+};
+template <typename T>
+__global__ __launch_bounds__(256) void qkv_norm_kernel(QkvNormArgs a) {
+    __shared__ float part[4];
+    const int64_t t = blockIdx.x;
+    const int tid = threadIdx.x;
+    const T* row = (const T*)a.p + t * a.p_stride;
+    const int nq = a.H * a.D, nk = a.G * a.D;
+    const int kind = blockIdx.y;                      // 0: q; 1: k and v
+    const T* src = row + (kind ? a.k_off : a.q_off);
+    const int n = kind ? nk : nq;
+    float ss = 0.0f;
+    for (int i = tid; i < n; i += 256) { const float f = ld(src + i); ss += f * f; }
+    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)n + a.eps);
+    if (kind == 0) {
+        T* dst = (T*)a.q + t * a.H * a.Dp;
+        for (int i = tid; i < a.H * a.Dp; i += 256) {
+            const int h = i / a.Dp, d = i - h * a.Dp, e = h * a.D + d;
+            st(dst + i, d < a.D ? ld(src + e) * inv * a.qw[e] : 0.0f);
+        }
+        return;
+    }
+    int64_t kstep = a.Dp, vstep = a.Dvp, k0 = t * a.G * a.Dp, v0 = t * a.G * a.Dvp;
+    if (a.slots) {
+        const int slot = a.slots[t], cap = a.keep + a.size, r = ring_slot(a.seen[2 * slot], a.keep, a.size);
+        kstep = (int64_t)cap * a.Dp; vstep = (int64_t)cap * a.Dvp;
+        k0 = (int64_t)slot * a.G * kstep + (int64_t)r * a.Dp; v0 = (int64_t)slot * a.G * vstep + (int64_t)r * a.Dvp;
+    }
+    for (int i = tid; i < a.G * a.Dp; i += 256) {
+        const int g = i / a.Dp, d = i - g * a.Dp, e = g * a.D + d;
+        st((T*)a.k + k0 + g * kstep + d, d < a.D ? ld(src + e) * inv * a.kw[e] : 0.0f);
+    }
+    const T* vs = row + a.v_off;
+    for (int i = tid; i < a.G * a.Dvp; i += 256) {
+        const int g = i / a.Dvp, d = i - g * a.Dvp;
+        st((T*)a.v + v0 + g * vstep + d, d < a.Dv ? ld(vs + g * a.Dv + d) : 0.0f);
+    }
+}
+
+// ---- a prompt's surviving rows into the ring -----------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void ring_store_kernel(const T* k, const T* v, const int32_t* cu, const int32_t* slots, const int32_t* seen,
+                                                         T* rk, T* rv, int G, int Dp, int Dvp, int keep, int size) {
+    const int b = blockIdx.y, slot = slots[b], t0 = cu[b], len = cu[b + 1] - t0, past = seen[2 * slot];
+    const int i = blockIdx.x;                          // token of the portion
+    if (i >= len) return;
+    const int pos = past + i;
+    if (pos >= keep && pos < past + len - size) return;     // a later token takes its slot
+    const int cap = keep + size, r = ring_slot(pos, keep, size);
+    const T* ks = k + (int64_t)(t0 + i) * G * Dp;
+    const T* vs = v + (int64_t)(t0 + i) * G * Dvp;
+    for (int e = threadIdx.x; e < G * Dp; e += 256) {
+        const int g = e / Dp, d = e - g * Dp;
+        rk[(((int64_t)slot * G + g) * cap + r) * Dp + d] = ks[e];
+    }
+    for (int e = threadIdx.x; e < G * Dvp; e += 256) {
+        const int g = e / Dvp, d = e - g * Dvp;
+        rv[(((int64_t)slot * G + g) * cap + r) * Dvp + d] = vs[e];
+    }
+}
+
+// ---- behind a recurrence: rms per head, weight, sigmoid gate -------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* o, const T* g, int64_t g_stride, const float* w, T* out, int64_t units, int H, int Dv, float eps) {
+    const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (unit >= units) return;
+    const int64_t t = unit / H;
+    const int h = (int)(unit - t * H), lane = threadIdx.x & 63;
+    const float* src = o + unit * Dv;
+    const T* gr = g + t * g_stride + h * Dv;
+    float ss = 0.0f;
+    for (int i = lane; i < Dv; i += 64) ss += src[i] * src[i];
+    const float inv = 1.0f / sqrtf(wave_sum_f(ss) / (float)Dv + eps);
+    for (int i = lane; i < Dv; i += 64) st(out + unit * Dv + i, src[i] * inv * w[h * Dv + i] * sigmoid_f(ld(gr + i)));
+}
+
+__global__ void advance_kernel(int32_t* seen, const int32_t* slots, const int32_t* cu, int batch) {
+    const int b = blockIdx.x * 64 + threadIdx.x;
+    if (b >= batch) return;
+    const int slot = slots[b];
+    seen[2 * slot] += cu[b + 1] - cu[b];
+    seen[2 * slot + 1] += 1;
+}
+
+}  // namespace trimkv
+
+using namespace trimkv;
+
+extern "C" const char* trimkv_hybrid_last_error(void) { return err_buf(); }
+
+extern "C" int trimkv_embed_scaled(const int64_t* ids, const void* table, float scale, float* x, void* xh, int tokens, int vocab, int width,
+                                   int x_stride, int dtype, void* stream) {
+    const char* fn = "trimkv_embed_scaled";
+    if (!ids || !table || !x) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (tokens <= 0 || vocab <= 0 || width <= 0 || x_stride < width) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d vocab=%d width=%d stride=%d", fn, tokens, vocab, width, x_stride);
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((embed_kernel<T>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, ids, (const T*)table, scale, x, (T*)xh, vocab, width, x_stride));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_linear_f32(const float* x, int64_t x_stride, const void* w, int64_t w_stride, float* out, int rows, int n, int k, int dtype, void* stream) {
+    const char* fn = "trimkv_linear_f32";
+    if (!x || !w || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (rows <= 0 || n <= 0 || k <= 0 || k % 4 || x_stride < k || w_stride < k || x_stride % 4 || w_stride % 8)
+        return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes rows=%d n=%d k=%d strides %lld %lld", fn, rows, n, k, (long long)x_stride, (long long)w_stride);
+    if (((uintptr_t)x | (uintptr_t)w) & 15) return fail(TRIMKV_ERR_SHAPE, "%s: x and w must be 16-byte aligned", fn);
+    hipStream_t st_ = (hipStream_t)stream;
+    if (dtype == TRIMKV_BF16 && k % 32 == 0) {
+        const bf16_t* wb = (const bf16_t*)w;
+        if (rows >= 2048 && n > 16)
+            hipLaunchKernelGGL((linear_f32_mfma_kernel<4, 4>), dim3((rows + 15) / 16, (n + 63) / 64), dim3(256), 0, st_, x, x_stride, wb, w_stride, out, rows, n, k);
+        else if (rows >= 2048)
+            hipLaunchKernelGGL((linear_f32_mfma_kernel<1, 4>), dim3((rows + 15) / 16, (n + 15) / 16), dim3(256), 0, st_, x, x_stride, wb, w_stride, out, rows, n, k);
+        else
+            hipLaunchKernelGGL((linear_f32_mfma_kernel<1, 16>), dim3((rows + 15) / 16, (n + 15) / 16), dim3(1024), 0, st_, x, x_stride, wb, w_stride, out, rows, n, k);
+        return launch_status(fn);
+    }
+    const int64_t units = (int64_t)rows * n;
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((linear_f32_kernel<T>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, st_, x, x_stride, (const T*)w, w_stride, out, units, n, k));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_residual_norm(const void* y, int64_t y_stride, const float* y_weight, int top, float* x, const float* w, void* xh,
+                                    int tokens, int width, int x_stride, float eps, int dtype, void* stream) {
+    const char* fn = "trimkv_residual_norm";
+    if (!y || !x || !w) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (tokens <= 0 || width <= 0 || width > 16384 || top < 1 || x_stride < width || y_stride < width)
+        return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d width=%d top=%d", fn, tokens, width, top);
+    if (!y_weight && top != 1) return fail(TRIMKV_ERR_SHAPE, "%s: several rows per token need weights", fn);
+    ResidualNormArgs a{y, y_stride, y_weight, top, x, w, xh, width, x_stride, eps};
+    const bool vec = width % 4 == 0 && x_stride % 4 == 0 && y_stride % 4 == 0 && !((((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)xh)) & 15);
+    const size_t lds = (size_t)width * 4;
+    HY_BY_DTYPE(dtype, T,
+        if (vec) hipLaunchKernelGGL((residual_norm_kernel<T, true>), dim3(tokens), dim3(256), lds, (hipStream_t)stream, a);
+        else hipLaunchKernelGGL((residual_norm_kernel<T, false>), dim3(tokens), dim3(256), lds, (hipStream_t)stream, a));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_rms_rows(const float* x, int x_stride, const int64_t* rows, const float* w, void* out, int count, int width, float eps, int dtype, void* stream) {
+    const char* fn = "trimkv_rms_rows";
+    if (!x || !w || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (count <= 0 || width <= 0 || x_stride < width) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes count=%d width=%d", fn, count, width);
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((rms_rows_kernel<T>), dim3(count), dim3(256), 0, (hipStream_t)stream, x, x_stride, rows, w, (T*)out, width, eps));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_qkv_norm(const void* proj, int64_t proj_stride, int q_off, int k_off, int v_off, const float* q_weight, const float* k_weight, float eps,
+                               int heads, int kv_heads, int dim, int vdim, int dim_stride, int vdim_stride, void* q, void* k, void* v,
+                               const int32_t* slots, const int32_t* seen, int keep_first, int window, int tokens, int dtype, void* stream) {
+    const char* fn = "trimkv_qkv_norm";
+    if (!proj || !q_weight || !k_weight || !q || !k || !v || (!slots != !seen)) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || dim_stride < dim || vdim_stride < vdim || (slots && (window <= 0 || keep_first < 0)))
+        return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d heads=%d kv_heads=%d dim=%d vdim=%d", fn, tokens, heads, kv_heads, dim, vdim);
+    QkvNormArgs a{proj, proj_stride, q_off, k_off, v_off, q_weight, k_weight, eps, heads, kv_heads, dim, vdim, dim_stride, vdim_stride, q, k, v, slots, seen, keep_first, window};
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((qkv_norm_kernel<T>), dim3(tokens, 2), dim3(256), 0, (hipStream_t)stream, a));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_ring_store(const void* k, const void* v, const int32_t* cu, const int32_t* slots, const int32_t* seen, void* ring_k, void* ring_v,
+                                 int batch, int max_len, int kv_heads, int dim_stride, int vdim_stride, int keep_first, int window, int dtype, void* stream) {
+    const char* fn = "trimkv_ring_store";
+    if (!k || !v || !cu || !slots || !seen || !ring_k || !ring_v) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (batch <= 0 || batch > 65535 || max_len <= 0 || kv_heads <= 0 || dim_stride <= 0 || vdim_stride <= 0 || keep_first < 0 || window <= 0)
+        return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes batch=%d max_len=%d kv_heads=%d keep=%d window=%d", fn, batch, max_len, kv_heads, keep_first, window);
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((ring_store_kernel<T>), dim3(max_len, batch), dim3(256), 0, (hipStream_t)stream,
+                                             (const T*)k, (const T*)v, cu, slots, seen, (T*)ring_k, (T*)ring_v, kv_heads, dim_stride, vdim_stride, keep_first, window));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int tokens, int heads, int vdim, float eps, int dtype, void* stream) {
+    const char* fn = "trimkv_head_norm_gate";
+    if (!o || !gate || !w || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (tokens <= 0 || heads <= 0 || vdim <= 0) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d heads=%d vdim=%d", fn, tokens, heads, vdim);
+    const int64_t units = (int64_t)tokens * heads;
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((head_norm_gate_kernel<T>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_advance(int32_t* seen, const int32_t* slots, const int32_t* cu, int batch, void* stream) {
+    const char* fn = "trimkv_advance";
+    if (!seen || !slots || !cu) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    if (batch <= 0) return fail(TRIMKV_ERR_SHAPE, "%s: bad batch %d", fn, batch);
+    hipLaunchKernelGGL(advance_kernel, dim3((batch + 63) / 64), dim3(64), 0, (hipStream_t)stream, seen, slots, cu, batch);
+    return launch_status(fn);
+}

@@ -25,6 +25,7 @@ import torch
 
 from . import decoder_ops
 from .cache_utils import TrimKVCache
+from .hybrid_cache import HybridCache
 
 
 class GraphedDecoder:
@@ -35,21 +36,29 @@ class GraphedDecoder:
 
     ``model``: a ``TrimKVQwen3Model`` / ``TrimKVQwen3ForCausalLM`` (or the Llama / Phi-3 subclasses) with
     ``compress_memory`` on and the ``trimkv_hip`` attention; ``cache``: the dense ``TrimKVCache`` that holds the prompt.
+    A ``HybridForCausalLM`` over its ``HybridCache`` is replayed as well (by ``input_ids``; the sequences in the batch must
+    stay the same, else the step is captured anew).
     ``forward_kwargs`` are passed to every call of the model (e.g. ``logits_to_keep=1``)."""
 
     def __init__(self, model, cache: TrimKVCache, gate_on_side_stream: bool = False, **forward_kwargs):
         cfg = model.config
-        if type(cache) is not TrimKVCache:
-            raise TypeError("GraphedDecoder replays steps of the dense TrimKVCache only")
-        if not cfg.compress_memory:
-            raise ValueError("GraphedDecoder needs compress_memory: a cache that only grows has to move its slabs, which a graph cannot replay")
-        if cfg._attn_implementation != "trimkv_hip":
-            raise ValueError("GraphedDecoder needs the trimkv_hip attention (lengths are read on the device)")
         self.model, self.cache, self.kwargs = model, cache, forward_kwargs
-        self.memory_size, self.buffer_size = cfg.memory_size, cfg.buffer_size
-        cache.fuse_decode_append = True
-        cache.begin_device_steps(self.memory_size, self.buffer_size)
-        dev = cache._slabs[0].k.device
+        self.hybrid = isinstance(cache, HybridCache)
+        if self.hybrid:
+            self.memory_size = self.buffer_size = 0
+            cache.begin_device_steps()
+            dev = cache.device
+        else:
+            if type(cache) is not TrimKVCache:
+                raise TypeError("GraphedDecoder replays steps of the dense TrimKVCache and of the HybridCache only")
+            if not cfg.compress_memory:
+                raise ValueError("GraphedDecoder needs compress_memory: a cache that only grows has to move its slabs, which a graph cannot replay")
+            if cfg._attn_implementation != "trimkv_hip":
+                raise ValueError("GraphedDecoder needs the trimkv_hip attention (lengths are read on the device)")
+            self.memory_size, self.buffer_size = cfg.memory_size, cfg.buffer_size
+            cache.fuse_decode_append = True
+            cache.begin_device_steps(self.memory_size, self.buffer_size)
+            dev = cache._slabs[0].k.device
         self.device = dev
         self.position = torch.zeros(1, dtype=torch.int64, device=dev)   # cache_position of the step's token
         self.stream = torch.cuda.Stream(device=dev)
@@ -59,9 +68,12 @@ class GraphedDecoder:
         self.out = None
         self.calls = 0
         self._epoch = -1
-        self._fork_gate = bool(gate_on_side_stream) and cfg.retention_gate == "rg"
+        self._slots = None
+        self._fork_gate = bool(gate_on_side_stream) and getattr(cfg, "retention_gate", None) == "rg"
 
     def _forward(self):
+        if self.hybrid:
+            return self.model(input_ids=self.static_in, past_key_values=self.cache, **self.kwargs)
         arg = {"input_ids": self.static_in} if self.by_ids else {"inputs_embeds": self.static_in}
         return self.model(**arg, past_key_values=self.cache, cache_position=self.position, **self.kwargs)
 
@@ -77,6 +89,8 @@ class GraphedDecoder:
     def __call__(self, input_ids: Optional[torch.Tensor] = None, inputs_embeds: Optional[torch.Tensor] = None):
         if (input_ids is None) == (inputs_embeds is None):
             raise ValueError("pass exactly one of input_ids or inputs_embeds")
+        if self.hybrid and input_ids is None:
+            raise ValueError("GraphedDecoder: a hybrid decoder takes input_ids")
         x = input_ids if input_ids is not None else inputs_embeds
         if x.shape[1] != 1:
             raise ValueError("GraphedDecoder takes one new token per sequence")
@@ -94,6 +108,8 @@ class GraphedDecoder:
             # some decoder's parameters were moved into another buffer since the capture (a module replaced, a model moved):
             # the recorded addresses may be stale.  This step runs eagerly, the next one is captured anew.
             self.graph, self.out, self.calls = None, None, 1
+        if self.hybrid and self._slots != tuple(cache.active):
+            self._slots, self.graph, self.out, self.calls = tuple(cache.active), None, None, 1     # other sequences: other slots in the launches
         if self.calls == 1:
             # eager, on the capture's stream: first-use allocations (workspaces, address tables, library handles) happen here
             cur = torch.cuda.current_stream(self.device)

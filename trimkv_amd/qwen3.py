@@ -13,8 +13,6 @@ generation utilities beyond greedy decoding are out of scope.
 from __future__ import annotations
 
 import dataclasses
-import glob
-import json
 import os
 from dataclasses import dataclass
 from types import SimpleNamespace
@@ -28,6 +26,8 @@ from . import decoder_ops
 from .attn import get_attention_interface
 from .cache_utils import LazyLogBeta, TrimKVCache
 from .gate import RetentionGate, RetentionGate2, RetentionGate3
+from .generation import GreedyGeneration
+from .registry import load_checkpoint_tensors, read_config
 
 
 @dataclass
@@ -454,24 +454,7 @@ class TrimKVQwen3Model(nn.Module):
         return SimpleNamespace(last_hidden_state=hidden_states, past_key_values=past_key_values)
 
 
-def _load_checkpoint_tensors(directory: str) -> dict:
-    """All tensors of a local HF checkpoint directory: ``*.safetensors`` shards, else ``pytorch_model*.bin`` read with
-    ``weights_only=True`` (nothing in the files is executed)."""
-    shards = sorted(glob.glob(os.path.join(directory, "*.safetensors")))
-    state = {}
-    if shards:
-        from safetensors.torch import load_file
-        for f in shards:
-            state.update(load_file(f))
-        return state
-    for f in sorted(glob.glob(os.path.join(directory, "pytorch_model*.bin"))):
-        state.update(torch.load(f, map_location="cpu", weights_only=True))
-    if not state:
-        raise FileNotFoundError(f"no *.safetensors or pytorch_model*.bin under {directory}")
-    return state
-
-
-class TrimKVQwen3ForCausalLM(nn.Module):
+class TrimKVQwen3ForCausalLM(GreedyGeneration, nn.Module):
     model_cls = TrimKVQwen3Model
     config_cls = TrimKVQwen3Config
 
@@ -488,17 +471,13 @@ class TrimKVQwen3ForCausalLM(nn.Module):
         if download_from != "local":
             raise ValueError(f"Unsupported download_from value: {download_from}")
         path = pretrained_model_name_or_path
-        if not os.path.isdir(path):
-            raise ValueError(f"Path {path} does not exist.")
-        with open(os.path.join(path, "config.json")) as f:
-            raw = json.load(f)
-        config = cls.config_cls.from_dict(raw, **kwargs)
+        config = cls.config_cls.from_dict(read_config(path), **kwargs)
         base = config.base_model if (load_trimkv_weights and config.base_model) else path
         if not os.path.isdir(base):
             raise ValueError(f"base model {base!r} is not a local directory (nothing is downloaded here)")
         config.base_model = base
         model = cls(config)
-        state = _load_checkpoint_tensors(base)
+        state = load_checkpoint_tensors(base)
         if config.tie_word_embeddings and "lm_head.weight" not in state:
             state["lm_head.weight"] = state["model.embed_tokens.weight"]
         gate_keys = [k for k in model.state_dict() if any(t in k for t in config.trainable_params.split("|"))]
@@ -538,32 +517,3 @@ class TrimKVQwen3ForCausalLM(nn.Module):
         if logits_to_keep:
             h = h[:, -logits_to_keep:]
         return SimpleNamespace(logits=self.lm_head(h), past_key_values=out.past_key_values)
-
-    @torch.no_grad()
-    def generate(self, input_ids: torch.Tensor, max_new_tokens: int, past_key_values=None, prefill_chunk: int = 0,
-                 use_graph: bool = False):
-        """Greedy decoding.  ``prefill_chunk`` > 0 streams the prompt in chunks of that many tokens, evicting after
-        each (the long-prompt mode of the reference's examples); returns prompt + new tokens.  ``use_graph``: the decode
-        steps are captured in a HIP graph once and replayed (``trimkv_amd.graphed.GraphedDecoder``; dense cache with
-        ``compress_memory`` only); the cache goes back to host-sized launches when the call returns."""
-        chunk = prefill_chunk or input_ids.shape[1]
-        out = None
-        for s in range(0, input_ids.shape[1], chunk):
-            out = self(input_ids[:, s:s + chunk], past_key_values=past_key_values, logits_to_keep=1)
-            past_key_values = out.past_key_values
-        step, graphed = self, None
-        if use_graph and max_new_tokens > 1:
-            from .graphed import GraphedDecoder
-            graphed = GraphedDecoder(self, past_key_values, logits_to_keep=1)
-            step = lambda ids, **_: graphed(input_ids=ids)
-        tokens = [input_ids]
-        try:
-            for i in range(max_new_tokens):
-                nxt = out.logits[:, -1].argmax(-1, keepdim=True)
-                tokens.append(nxt)
-                if i + 1 < max_new_tokens:
-                    out = step(nxt, past_key_values=past_key_values, logits_to_keep=1)
-        finally:
-            if graphed is not None:
-                graphed.close()
-        return torch.cat(tokens, dim=1)
