@@ -1,0 +1,220 @@
+"""Fusitar end to end on the GPU against the plain oracle: prompts, portions, decoding, unequal batches, slots that are used
+again, greedy generation through the framework's own entry point (eager and replayed), loading from disk, trace replay."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+from safetensors.torch import save_file
+
+from trimkv_amd import registry
+from trimkv_amd.graphed import GraphedDecoder
+from tests.hybrid_util import DEV, assert_rows, attention, build, config, mlstm, moe, oracle, tokens, weights
+
+pytestmark = pytest.mark.gpu
+DTYPES = [torch.float32, torch.bfloat16]
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+CONFIGS = {
+    "mixed": config([attention(mlp=moe()), mlstm(mlp=moe(experts=8, top=3, ff=24, count=2, keep=1)), mlstm(), attention(heads=2, kv_heads=2, dim=16, vdim=16, size=20, keep_first=0, mlp=moe())]),
+    "recurrent_first": config([mlstm(heads=1, dim=64, vdim=64, gate_cap=15.0, mlp=moe(experts=4, top=1, ff=8, count=1, keep=1)), attention(heads=6, kv_heads=1, dim=48, vdim=64, size=33, keep_first=65, mlp=None)],
+                              vocab=130, width=128, eps=1e-6, scale=1.0),
+    "attention_only": config([attention(heads=8, kv_heads=4, dim=64, vdim=32, size=70, keep_first=1)], vocab=51, width=200),
+    "recurrent_only": config([mlstm(heads=5, dim=20, vdim=12)], vocab=33, width=60),
+}
+
+
+def packed_step(model, cache, parts, slots):
+    flat = torch.tensor([t for p in parts for t in p], device=DEV)
+    out = model(flat, past_key_values=cache, lengths=[len(p) for p in parts], slots=slots)
+    return out.logits.reshape(-1, out.logits.shape[-1]).split([len(p) for p in parts])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_prompt_portions_and_decode(name, dtype):
+    cfg = CONFIGS[name]
+    w = weights(cfg)
+    model = build(cfg, w, dtype)
+    toks = tokens(cfg, 190)
+    want = oracle(cfg, w, toks)
+    whole = model(torch.tensor([toks], device=DEV)).logits[0]
+    assert_rows(whole, want, dtype, "whole prompt")
+    for cuts in ([2] * 10 + [170], [64, 65, 1, 60], [1] * 40 + [150], [120] + [1] * 70):
+        cache, rows, at = model.new_cache(), [], 0
+        (slot,) = cache.allocate(1)
+        for n in cuts:
+            rows.append(packed_step(model, cache, [toks[at:at + n]], [slot])[0])
+            at += n
+        assert_rows(torch.cat(rows), want, dtype, f"cut {cuts[:3]}")
+        assert cache.get_seq_length() == 190 and cache.seen[slot].tolist() == [190, len(cuts)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_unequal_batches_and_slots_used_again(dtype):
+    cfg = CONFIGS["mixed"]
+    w = weights(cfg, 3)
+    model = build(cfg, w, dtype)
+    cache = model.new_cache(2)
+    seqs = {i: tokens(cfg, n, seed=10 + i) for i, n in enumerate((1 + 12, 40 + 5, 23 + 30, 97 + 30, 9 + 11))}
+    want = {i: oracle(cfg, w, s) for i, s in seqs.items()}
+    rows = {i: [] for i in seqs}
+
+    def run(ids, counts, slots):
+        parts = []
+        for i, n in zip(ids, counts):
+            at = sum(r.shape[0] for r in rows[i])
+            parts.append(seqs[i][at:at + n])
+        for i, r in zip(ids, packed_step(model, cache, parts, [slots[i] for i in ids])):
+            rows[i].append(r)
+
+    slots = {i: cache.allocate(1)[0] for i in range(4)}            # grows past the two slots it was made with
+    run([0, 1, 2, 3], [1, 40, 23, 97], slots)
+    for _ in range(5):
+        run([3, 1, 0, 2], [1] * 4, slots)                           # another order of the same batch
+    cache.release([slots[1]])
+    for _ in range(7):
+        run([0, 2, 3], [1] * 3, slots)
+    cache.release([slots[0]])
+    slots[4] = cache.allocate(1)[0]
+    assert slots[4] in (slots[0], slots[1]) or slots[4] >= 4
+    run([4], [9], slots)
+    for _ in range(11):
+        run([2, 4, 3], [1] * 3, slots)
+    for _ in range(7):
+        run([3, 2], [1] * 2, slots)
+    for i in seqs:
+        assert_rows(torch.cat(rows[i]), want[i], dtype, f"sequence {i}")
+
+
+def test_every_slot_is_used_again_and_again():
+    cfg = CONFIGS["mixed"]
+    w = weights(cfg, 4)
+    model = build(cfg, w, torch.float32)
+    cache = model.new_cache(2)
+    for turn in range(4):
+        slots = cache.allocate(2)
+        a, b = tokens(cfg, 30 + turn, 50 + turn), tokens(cfg, 17, 60 + turn)
+        first = packed_step(model, cache, [a[:20], b[:9]], slots)
+        rest = [packed_step(model, cache, [[a[20 + k]], [b[9 + k]]], slots) for k in range(8)]
+        assert_rows(torch.cat([first[0]] + [r[0] for r in rest]), oracle(cfg, w, a)[:28], torch.float32, f"turn {turn}")
+        assert_rows(torch.cat([first[1]] + [r[1] for r in rest]), oracle(cfg, w, b), torch.float32, f"turn {turn}")
+        cache.release(slots)
+    assert cache.num_slots == 2
+
+
+def test_long_decode():
+    cfg = CONFIGS["mixed"]
+    w = weights(cfg, 5)
+    model = build(cfg, w, torch.float32)
+    toks = tokens(cfg, 420, 7)
+    cache = model.new_cache()
+    slot = cache.allocate(1)
+    rows = [packed_step(model, cache, [toks[:20]], slot)[0]] + [packed_step(model, cache, [[t]], slot)[0] for t in toks[20:]]
+    assert_rows(torch.cat(rows), oracle(cfg, w, toks), torch.float32)
+
+
+def greedy(cfg, w, prompt, n):
+    out = list(prompt)
+    margins = []
+    for _ in range(n):
+        last = oracle(cfg, w, out)[-1]
+        two = last.topk(2)
+        margins.append(float(two.values[0] - two.values[1]))
+        out.append(int(two.indices[0]))
+    return out, min(margins)
+
+
+@pytest.mark.parametrize("use_graph", [False, True])
+@pytest.mark.parametrize("chunk", [0, 2, 13])
+def test_generate(use_graph, chunk):
+    cfg = CONFIGS["mixed"]
+    w = weights(cfg, 6)
+    model = build(cfg, w, torch.float32)
+    prompts = [tokens(cfg, 26, 70), tokens(cfg, 26, 71)]
+    got = model.generate(torch.tensor(prompts, device=DEV), 14, prefill_chunk=chunk, use_graph=use_graph).tolist()
+    for p, g in zip(prompts, got):
+        want, margin = greedy(cfg, w, p, 14)
+        assert margin > 1e-3, "choose another seed: the oracle's choice is too close"
+        assert g == want
+    # unequal prompts, padded on the right: each as alone
+    uneq = [tokens(cfg, n, 80 + n) for n in (3, 31, 12)]
+    ids = torch.zeros(3, 31, dtype=torch.int64, device=DEV)
+    for b, p in enumerate(uneq):
+        ids[b, :len(p)] = torch.tensor(p, device=DEV)
+    together = model.generate(ids, 9, prefill_chunk=chunk, use_graph=use_graph, lengths=[len(p) for p in uneq])
+    for p, g in zip(uneq, together):
+        assert g.tolist() == greedy(cfg, w, p, 9)[0]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_replayed_steps_equal_eager_ones(dtype):
+    """Several replays with eager work on another cache between them; sequences that end make the step be captured anew."""
+    cfg = CONFIGS["mixed"]
+    w = weights(cfg, 8)
+    model = build(cfg, w, dtype)
+    seqs = [tokens(cfg, 40, 90 + b) for b in range(3)]
+    eager, replayed = model.new_cache(3), model.new_cache(3)
+    for cache in (eager, replayed):
+        cache.allocate(3)
+        packed_step(model, cache, [s[:10 + b] for b, s in enumerate(seqs)], cache.active)
+    dec = GraphedDecoder(model, replayed, logits_to_keep=1)
+    for k in range(20):
+        if k == 12:
+            for cache in (eager, replayed):
+                cache.release([cache.active[1]])
+            seqs.pop(1)
+            dec.close()
+            dec = GraphedDecoder(model, replayed, logits_to_keep=1)
+        ids = torch.tensor([[s[20 + k]] for s in seqs], device=DEV)
+        a = model(ids, past_key_values=eager, logits_to_keep=1).logits
+        torch.cuda.synchronize()
+        b = dec(input_ids=ids).logits
+        assert torch.equal(a, b), k
+    dec.close()
+    assert replayed.tokens_seen == eager.tokens_seen and torch.equal(replayed.seen, eager.seen)
+
+
+def test_batch_select_copies_and_frees():
+    cfg = CONFIGS["mixed"]
+    w = weights(cfg, 9)
+    model = build(cfg, w, torch.float32)
+    cache = model.new_cache()
+    seqs = [tokens(cfg, 20, 100 + b) for b in range(3)]
+    cache.allocate(3)
+    packed_step(model, cache, seqs, cache.active)
+    cache.batch_select_indices(torch.tensor([2, 0, 2]))
+    tails = [tokens(cfg, 6, 110 + b) for b in range(3)]
+    rows = [packed_step(model, cache, [[t[k]] for t in tails], cache.active) for k in range(6)]
+    for b, src in enumerate((2, 0, 2)):
+        assert_rows(torch.cat([r[b] for r in rows]), oracle(cfg, w, seqs[src] + tails[b])[20:], torch.float32)
+
+
+def test_from_disk_and_trace_replay(tmp_path):
+    """config.json + safetensors -> registry -> logits, and the same requests through bin/trace_run."""
+    cfg = CONFIGS["recurrent_first"]
+    w = weights(cfg, 12)
+    (tmp_path / "m").mkdir()
+    (tmp_path / "out").mkdir()
+    (tmp_path / "m" / "config.json").write_text(json.dumps(cfg))
+    save_file(w, str(tmp_path / "m" / "model.safetensors"))
+    model = registry.from_pretrained(str(tmp_path / "m"), torch_dtype=torch.float32).to(DEV)
+    a, b = tokens(cfg, 30, 120), tokens(cfg, 12, 121)
+    wa, wb = oracle(cfg, w, a), oracle(cfg, w, b)
+    assert_rows(model(torch.tensor([a], device=DEV)).logits[0], wa, torch.float32)
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": a[:25], "want": [0, 24]}, {"id": "y", "tokens": b[:11], "want": []}], "end": []},
+             {"step": 1, "entries": [{"id": "y", "tokens": b[11:], "want": [0]}, {"id": "x", "tokens": a[25:26], "want": [0]}], "end": ["y"]},
+             {"step": 2, "entries": [{"id": "x", "tokens": a[26:27], "want": []}], "end": ["x"]},
+             {"step": 3, "entries": [{"id": "z", "tokens": b, "want": list(range(12))}], "end": ["z"]}]
+    proc = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path / "m"), "--dtype", "float32", "--out", str(tmp_path / "out"),
+                           "--max-tokens", "64"], input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=100)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert [l for l in proc.stdout.splitlines() if l.startswith("done")] == [f"done {i}" for i in range(4)]
+    read = lambda i: torch.from_numpy(np.fromfile(tmp_path / "out" / f"{i}.f32", "<f4").reshape(-1, cfg["vocab"]))
+    assert_rows(read(0), wa[[0, 24]], torch.float32)
+    assert_rows(read(1), torch.stack([wb[11], wa[25]]), torch.float32)
+    assert not (tmp_path / "out" / "2.f32").exists()
+    assert_rows(read(3), wb, torch.float32)

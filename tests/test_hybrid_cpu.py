@@ -1,0 +1,139 @@
+"""CPU checks of the hybrid decoders: ABI of libtrimkv_hybrid.so, configuration and registry, loading, refusal to run without a
+GPU, and the oracle's own mechanisms on cases small enough to work out by hand."""
+import ctypes
+import json
+import math
+import os
+import re
+
+import pytest
+import torch
+from safetensors.torch import save_file
+
+from oracle import hybrid_ref as ref
+from trimkv_amd import _lib, registry
+from trimkv_amd.fusitar import FusitarConfig, FusitarForCausalLM
+from tests.hybrid_util import attention, config, mlstm, moe, weights
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+TEXT = re.sub(r"/\*.*?\*/", "", open(os.path.join(ROOT, "include", "trimkv_hybrid.h")).read(), flags=re.S)
+
+
+def test_header_binding_and_library_agree():
+    declared = sorted(set(re.findall(r"\b(trimkv_[a-z0-9_]+)\s*\(", TEXT)))
+    assert sorted(_lib.HYBRID_SIGNATURES) == declared
+    lib = ctypes.CDLL(_lib.HYBRID_LIB_PATH)
+    for name, (_, argtypes) in _lib.HYBRID_SIGNATURES.items():
+        assert hasattr(lib, name), name
+        params = re.search(r"\b%s\s*\(([^;]*?)\)\s*;" % name, TEXT, flags=re.S).group(1).strip()
+        want = [] if params in ("", "void") else [p.strip() for p in params.split(",")]
+        kinds = [_lib.C.c_void_p if "*" in p else _lib.C.c_int64 if p.startswith("int64_t") else _lib.C.c_float if p.startswith("float") else _lib.C.c_int for p in want]
+        assert kinds == argtypes, name
+
+
+def test_bad_arguments_are_refused_without_a_launch():
+    lib = _lib.load_hybrid()
+    one = ctypes.c_void_p(16)
+    assert lib.trimkv_embed_scaled(None, one, 1.0, one, None, 1, 4, 8, 64, _lib.F32, None) == -1
+    assert lib.trimkv_embed_scaled(one, one, 1.0, one, None, 1, 4, 8, 64, _lib.F16, None) == -3
+    assert lib.trimkv_linear_f32(one, 64, one, 64, one, 1, 3, 62, _lib.F32, None) == -2
+    assert b"bad sizes" in lib.trimkv_hybrid_last_error()
+    win = lambda H=4, G=2, D=16, Dp=16, keep=1, size=4, dt=_lib.BF16: lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, H, G, D, D, Dp, Dp, keep, size, 1.0, 1, None, dt, None)
+    assert win(H=5) == -2 and win(Dp=12, D=12) == -2 and win(size=0) == -2 and win(keep=-1) == -2 and win(D=520, Dp=520) == -6 and win(dt=7) == -3
+    assert lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, 4, 2, 16, 16, 16, 16, 1, 4, 1.0, 3, None, _lib.BF16, None) == -5
+    assert lib.trimkv_moe_route(one, one, one, one, 1, 8, 5, 2, 1, None) == -2          # one open group of four cannot give five
+    assert lib.trimkv_moe_route(one, one, one, one, 1, 9, 2, 2, 1, None) == -2
+    assert lib.trimkv_moe_gemm(one, 64, one, one, 64, one, one, one, 4, 2, 32, 1, 64, 64, 64, 1, _lib.BF16, None) == -2
+    assert lib.trimkv_mlstm(one, 64, 0, 8, 16, one, one, one, 1.0, one, one, one, one, one, one, 1, 1, 1, 513, 8, 1, 1.0, None, _lib.F32, None) == -6
+    assert lib.trimkv_window_decode_splits(64, 8, 4096) >= 1 and lib.trimkv_window_decode_splits(1, 1, 64) == 1
+    assert lib.trimkv_mlstm_workspace(1, 1, 4, 64, 64, _lib.BF16) == 0
+
+
+GOOD = config([attention(mlp=moe()), mlstm()])
+
+
+def test_configuration_is_checked():
+    cfg = FusitarConfig.from_dict(GOOD)
+    assert (cfg.vocab_size, cfg.hidden_size, cfg.num_hidden_layers, cfg.norm_eps) == (97, 72, 2, 2e-5)
+    for layer, text in ((attention(heads=5), "do not divide"), (dict(attention(), type="other"), "unknown mixer"), (attention(size=0), "bad window"),
+                        (attention(mlp=moe(experts=7)), "cannot choose"), (attention(mlp=moe(top=5)), "cannot choose"), (attention(mlp=dict(moe(), kind="x")), "unknown feed-forward"),
+                        ({"type": "mlstm", "mixer": {"heads": 1, "dim": 8, "vdim": 8}, "mlp": None}, "lacks")):
+        with pytest.raises(ValueError, match=text):
+            FusitarConfig.from_dict(dict(GOOD, layers=[layer]))
+
+
+def test_registry_finds_every_family():
+    assert registry.model_class(GOOD) is FusitarForCausalLM
+    for name, (module, cls) in registry.MODELS.items():
+        assert registry.model_class({"architectures": [name]}).__name__ == cls
+    with pytest.raises(ValueError, match="no model for architecture"):
+        registry.model_class({"architecture": "Nothing"})
+
+
+def test_loading_fills_every_parameter_and_refuses_what_does_not_fit(tmp_path):
+    w = weights(GOOD)
+    (tmp_path / "config.json").write_text(json.dumps(GOOD))
+    save_file(w, str(tmp_path / "model.safetensors"))
+    model = registry.from_pretrained(str(tmp_path), torch_dtype=torch.float32)
+    for name, t in model.tensors().items():
+        assert torch.equal(t, w[name].float()), name
+    # padding stays zero: kernels read it
+    assert not model.model.layers[0].mlp.up[:, 40:].any() and not model.model.layers[0].mlp.down[:, :, 40:].any()
+    for change in (lambda d: d.pop("l1.mix.f.b"), lambda d: d.update(extra=torch.zeros(1)), lambda d: d.update({"l0.norm1": torch.zeros(71)})):
+        bad = dict(w)
+        change(bad)
+        with pytest.raises(ValueError):
+            model.load_tensors(bad)
+    with pytest.raises(ValueError, match="bfloat16 or float32"):
+        FusitarForCausalLM(FusitarConfig.from_dict(GOOD), torch.float16)
+
+
+def test_no_cpu_path():
+    model = FusitarForCausalLM(FusitarConfig.from_dict(GOOD))
+    with pytest.raises(_lib.TrimKVLibraryError, match="GPU only"):
+        model(torch.tensor([[1, 2]]))
+    with pytest.raises(_lib.TrimKVLibraryError, match="GPU only"):
+        model.new_cache()
+
+
+# ---- the oracle on cases worked out by hand --------------------------------------------------------------
+def test_oracle_window():
+    seen = [[j for j in range(8) if ref.window_visible(i, j, 3, 2)] for i in range(8)]
+    assert seen[0] == [0] and seen[3] == [0, 1, 2, 3] and seen[7] == [0, 1, 5, 6, 7]
+    T = 8
+    q = torch.zeros(T, 1, 1, dtype=torch.float64)
+    v = torch.arange(T, dtype=torch.float64).view(T, 1, 1)
+    out = ref.window_attention(q, q, v, 1.0, 3, 2).flatten()
+    assert out.tolist() == pytest.approx([sum(s) / len(s) for s in seen])
+    # sensitive to a window and to a kept prefix that are one off
+    assert not torch.allclose(out, ref.window_attention(q, q, v, 1.0, 4, 2).flatten()) and not torch.allclose(out, ref.window_attention(q, q, v, 1.0, 3, 1).flatten())
+
+
+def test_oracle_mlstm_first_steps():
+    one = torch.ones(1, 1, 1, dtype=torch.float64)
+    li, lf = torch.tensor([[math.log(0.5)], [math.log(3.0)]], dtype=torch.float64), torch.tensor([[math.log(0.25)], [math.log(0.5)]], dtype=torch.float64)
+    out, (S, n, m) = ref.mlstm_scan(torch.cat([one, one]), torch.cat([one, 2 * one]), torch.cat([4 * one, 5 * one]), li, lf)
+    # unscaled: S1 = 0.5 * 4, n1 = 0.5; m1 = max(log .25 + 0, log .5) = log .5, so S = 4, n = 1, floor exp(-m1) = 2
+    assert out[0].item() == pytest.approx(4 / (2 + 1e-6))
+    # S2 = 0.5 * 2 + 3 * 2 * 5 = 31, n2 = 0.25 + 6 = 6.25, m2 = log 3
+    assert m.item() == pytest.approx(math.log(3)) and S.item() == pytest.approx(31 / 3) and n.item() == pytest.approx(6.25 / 3)
+    assert out[1].item() == pytest.approx((31 / 3) / (6.25 / 3 + 1e-6))
+    # the running maximum starts at 0: a first token with a tiny input gate is scaled down, not normalised away
+    out, (S, _, m) = ref.mlstm_scan(one, one, one, torch.tensor([[-9.0]], dtype=torch.float64), torch.tensor([[-1.0]], dtype=torch.float64))
+    assert m.item() == -1.0 and S.item() == pytest.approx(math.exp(-8.0))
+
+
+def test_oracle_router_by_hand():
+    z = torch.tensor([[0.0, 0.0, 2.0, -9.0, 1.0, 1.0]], dtype=torch.float64)
+    corr = torch.tensor([-0.1, -0.1, -0.9, 0.0, -0.7, -0.7], dtype=torch.float64)
+    s = torch.sigmoid(z[0])
+    ids, w = ref.choose_experts(z, corr, 2, 3, 1)                 # groups (0, 1), (2, 3), (4, 5); the first has the largest sum
+    assert sorted(ids[0].tolist()) == [0, 1] and torch.allclose(w, s[ids])
+    # all choice scores negative: closed groups must stay closed
+    ids, _ = ref.choose_experts(z, corr - 5.0, 2, 3, 1)
+    assert sorted(ids[0].tolist()) == [0, 1]
+
+
+def test_oracle_norm_has_eps_inside_the_root():
+    x = torch.tensor([3.0, 4.0], dtype=torch.float64)
+    assert torch.allclose(ref.rms(x, 12.5), x / 5.0)

@@ -94,7 +94,8 @@ HYBRID_SIGNATURES = {
     "trimkv_window_prefill": (_i, [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
     "trimkv_window_decode_splits": (_i, [_i, _i, _i]),
     "trimkv_window_decode": (_i, [_p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p, _i, _p]),
-    "trimkv_mlstm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _f, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
+    "trimkv_mlstm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _f, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _p, _i, _p]),
+    "trimkv_mlstm_workspace": (_i64, [_i, _i, _i, _i, _i, _i]),
     "trimkv_head_norm_gate": (_i, [_p, _p, _i64, _p, _p, _i, _i, _i, _f, _i, _p]),
     "trimkv_advance": (_i, [_p, _p, _p, _i, _p]),
     "trimkv_moe_route": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _i, _p]),

@@ -58,6 +58,7 @@ typedef float hy_f32x2 __attribute__((ext_vector_type(2)));
 typedef float hy_f32x4 __attribute__((ext_vector_type(4)));
 typedef float hy_f32x16 __attribute__((ext_vector_type(16)));
 typedef short hy_s16x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t hy_u32x2 __attribute__((ext_vector_type(2)));
 typedef uint32_t hy_u32x4 __attribute__((ext_vector_type(4)));
 #define HY_LDS __attribute__((address_space(3)))
 

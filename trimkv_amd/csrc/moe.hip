@@ -115,7 +115,7 @@ struct GroupedArgs {
 // squared ReLU of the up product; the down product passes
 template <bool UP> __device__ __forceinline__ float expert_act(float f) { return UP ? (f > 0.0f ? f * f : 0.0f) : f; }
 
-// General form: 16 rows x 64 outputs per workgroup, fp32 arithmetic.
+// fp32: 16 rows x 64 outputs per workgroup.
 template <typename T, bool UP>
 __global__ __launch_bounds__(256) void grouped_simple_kernel(GroupedArgs a) {
     __shared__ float xs[16][17];
@@ -144,6 +144,126 @@ __global__ __launch_bounds__(256) void grouped_simple_kernel(GroupedArgs a) {
     for (int y = 0; y < 4; ++y) {
         const int i = m0 + tm * 4 + y;
         if (i < mend && n0 + tn < a.n) st((T*)a.y + (UP ? (int64_t)i : (int64_t)a.order[i]) * a.ys + n0 + tn, expert_act<UP>(acc[y]));
+    }
+}
+
+// bf16, a handful of rows per expert (decode): 16 rows x 64 outputs per workgroup, 16 outputs per wavefront, operands straight
+// from memory (lane l: 8 consecutive k of weight row, or token row, l % 16 at k-group l / 16).  The launch is bound by the
+// stream of weights; UNROLL loads of them are in flight per lane.
+template <bool UP>
+__global__ __launch_bounds__(256) void grouped_skinny_kernel(GroupedArgs a) {
+    constexpr int UNROLL = 8;
+    if ((int)blockIdx.x >= a.tiles[0]) return;
+    const int e = a.tiles[1 + 2 * blockIdx.x], m0 = a.tiles[2 + 2 * blockIdx.x], mend = a.offsets[e + 1];
+    const int lane = threadIdx.x & 63, r = lane & 15, kg = lane >> 4, n0 = blockIdx.y * 64 + (threadIdx.x >> 6) * 16;
+    const int i = min(m0 + r, mend - 1);
+    const uint16_t* xr = (const uint16_t*)a.x + (UP ? (int64_t)(a.order[i] / a.top) : (int64_t)i) * a.xs + kg * 8;
+    const uint16_t* wr = (const uint16_t*)a.w + ((int64_t)e * a.np + n0 + r) * a.kp + kg * 8;
+    hy_f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    for (int k = 0; k < a.kp; k += 32 * UNROLL) {
+        hy_u32x4 wf[UNROLL], xf[UNROLL];
+#pragma unroll
+        for (int u = 0; u < UNROLL; ++u) wf[u] = __builtin_nontemporal_load((const hy_u32x4*)(wr + min(k + 32 * u, a.kp - 32)));
+#pragma unroll
+        for (int u = 0; u < UNROLL; ++u) {
+            xf[u] = *(const hy_u32x4*)(xr + min(k + 32 * u, a.kp - 32));
+            if (k + 32 * u >= a.kp) xf[u] = hy_u32x4{0u, 0u, 0u, 0u};
+        }
+#pragma unroll
+        for (int u = 0; u < UNROLL; ++u) acc[u & 1] = mfma16(__builtin_bit_cast(hy_bf16x8, wf[u]), __builtin_bit_cast(hy_bf16x8, xf[u]), acc[u & 1]);
+    }
+    // lane holds outputs n0 + 4 kg .. + 3 of row r
+    if (m0 + r >= mend) return;
+    uint16_t* y = (uint16_t*)a.y + (UP ? (int64_t)(m0 + r) : (int64_t)a.order[m0 + r]) * a.ys + n0 + 4 * kg;
+#pragma unroll
+    for (int v = 0; v < 4; ++v)
+        if (n0 + 4 * kg + v < a.n) y[v] = f32_to_bf16_bits(expert_act<UP>(acc[0][v] + acc[1][v]));
+}
+
+// bf16, many rows per expert (prompts): 128 rows x 128 outputs per workgroup, 64 x 64 per wavefront on 32x32x16 MFMAs, 64 k per
+// step through two LDS buffers filled by LDS-direct loads (whose lanes gather token rows as they please).  Row r keeps its
+// 16-byte piece c at c ^ ((r / 2) % 8), so that the rows of a fragment read fall on different banks.
+template <bool UP>
+__global__ __launch_bounds__(256) void grouped_big_kernel(GroupedArgs a, int n_tiles) {
+    extern __shared__ __attribute__((aligned(16))) char gb_lds[];
+    HY_LDS char* const lds3 = (HY_LDS char*)gb_lds;
+    const uint32_t lds0 = (uint32_t)(uintptr_t)lds3;
+    // an XCD takes a contiguous share of the row tiles and walks it in blocks of 4 row tiles x all outputs: the rows and the
+    // weights that neighbouring workgroups read stay in its L2
+    const int total = a.tiles[0], share = (total + 7) / 8, turn = blockIdx.x >> 3;
+    const int blk = turn / (4 * n_tiles), in = turn - blk * 4 * n_tiles;
+    const int first = blk * 4, rows_here = min(4, share - first);
+    if (rows_here <= 0) return;
+    const int rt_ = first + in % rows_here, nt = in / rows_here;
+    const int rt = (blockIdx.x & 7) * share + rt_;
+    if (nt >= n_tiles || rt >= total) return;
+    const int e = a.tiles[1 + 2 * rt], m0 = a.tiles[2 + 2 * rt], mend = a.offsets[e + 1], n0 = nt * 128;
+    const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane & 31, hl = lane >> 5;
+    const int wm = w & 1, wn = w >> 1;
+    const uint16_t* xp[4]; const uint16_t* wp[4];
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+        const int row = x * 32 + (tid >> 3), piece = (tid & 7) ^ ((row >> 1) & 7);
+        const int i = min(m0 + row, mend - 1);
+        xp[x] = (const uint16_t*)a.x + (UP ? (int64_t)(a.order[i] / a.top) : (int64_t)i) * a.xs + piece * 8;
+        wp[x] = (const uint16_t*)a.w + ((int64_t)e * a.np + min(n0 + row, a.np - 1)) * a.kp + piece * 8;
+    }
+    auto request = [&](int k, int buf) __attribute__((always_inline)) {
+        const uint32_t dst = lds0 + buf * 32768 + w * 1024;
+#pragma unroll
+        for (int x = 0; x < 4; ++x) load_to_lds16(xp[x] + k, dst + x * 4096);
+#pragma unroll
+        for (int x = 0; x < 4; ++x) load_to_lds16(wp[x] + k, dst + 16384 + x * 4096);
+    };
+    hy_f32x16 acc[2][2];
+#pragma unroll
+    for (int x = 0; x < 2; ++x)
+#pragma unroll
+        for (int y = 0; y < 2; ++y)
+#pragma unroll
+            for (int v = 0; v < 16; ++v) acc[x][y][v] = 0.0f;
+    const int sw = (j >> 1) & 7;
+    HY_LDS char* const xr = lds3 + (wm * 64 + j) * 128;
+    HY_LDS char* const wr = lds3 + 16384 + (wn * 64 + j) * 128;
+    request(0, 0);
+    const int steps = a.kp / 64;
+    for (int s = 0; s < steps; ++s) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        if (s + 1 < steps) request((s + 1) * 64, (s + 1) & 1);
+        const int off = (s & 1) * 32768;
+#pragma unroll
+        for (int ks = 0; ks < 4; ++ks) {
+            const int po = off + (((2 * ks + hl) ^ sw) << 4);
+            hy_bf16x8 xf[2], wf[2];
+#pragma unroll
+            for (int y = 0; y < 2; ++y) { xf[y] = *(const HY_LDS hy_bf16x8*)(xr + y * 4096 + po); wf[y] = *(const HY_LDS hy_bf16x8*)(wr + y * 4096 + po); }
+#pragma unroll
+            for (int x = 0; x < 2; ++x)
+#pragma unroll
+                for (int y = 0; y < 2; ++y) acc[x][y] = mfma32(wf[x], xf[y], acc[x][y]);
+        }
+    }
+    // acc[x][y]: outputs n0 + wn 64 + 32 x + 8 (v / 4) + 4 hl + v % 4 of row m0 + wm 64 + 32 y + j
+#pragma unroll
+    for (int y = 0; y < 2; ++y) {
+        const int i = m0 + wm * 64 + 32 * y + j;
+        if (i >= mend) continue;
+        uint16_t* yr = (uint16_t*)a.y + (UP ? (int64_t)i : (int64_t)a.order[i]) * a.ys;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+#pragma unroll
+            for (int c = 0; c < 4; ++c) {
+                const int n = n0 + wn * 64 + 32 * x + 8 * c + 4 * hl;
+                float f[4];
+#pragma unroll
+                for (int v = 0; v < 4; ++v) f[v] = expert_act<UP>(acc[x][y][4 * c + v]);
+                if (n + 3 < a.n && a.ys % 4 == 0) *(uint2*)(yr + n) = make_uint2(pack2(f[0], f[1]), pack2(f[2], f[3]));
+                else
+#pragma unroll
+                    for (int v = 0; v < 4; ++v)
+                        if (n + v < a.n) yr[n + v] = f32_to_bf16_bits(f[v]);
+            }
     }
 }
 
@@ -178,13 +298,22 @@ extern "C" int trimkv_moe_gemm(const void* x, int64_t x_stride, const void* w, v
     HY_CHECK_DTYPE(fn, dtype);
     if (rows <= 0 || experts <= 0 || top <= 0 || n <= 0 || n > n_padded || n_padded % 64 || k_padded <= 0 || k_padded % 64 || x_stride < k_padded || y_stride < n)
         return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes rows=%d experts=%d n=%d/%d k=%d", fn, rows, experts, n, n_padded, k_padded);
-    if (tile != 16) return fail(TRIMKV_ERR_SHAPE, "%s: row tiles of 16 (got %d)", fn, tile);
+    if (tile != 16 && !(tile == 128 && dtype == TRIMKV_BF16)) return fail(TRIMKV_ERR_SHAPE, "%s: row tiles of 16, or of 128 in bf16 (got %d)", fn, tile);
+    if (((uintptr_t)x | (uintptr_t)w | (uintptr_t)y) & 15 || x_stride % 8) return fail(TRIMKV_ERR_SHAPE, "%s: x, w and y must be 16-byte aligned", fn);
     GroupedArgs a{x, x_stride, w, y, y_stride, order, offsets, tiles, top, n, n_padded, k_padded};
     hipStream_t s = (hipStream_t)stream;
     const int most = rows < experts ? rows : (rows - experts) / tile + experts;     // no more row tiles than this
     const dim3 grid(most, n_padded / 64);
-    HY_BY_DTYPE(dtype, T,
-        if (up) hipLaunchKernelGGL((grouped_simple_kernel<T, true>), grid, dim3(256), 0, s, a);
-        else hipLaunchKernelGGL((grouped_simple_kernel<T, false>), grid, dim3(256), 0, s, a));
+    if (tile == 128) {
+        const int n_tiles = (n_padded + 127) / 128, blocks = 8 * (((most + 7) / 8 + 3) / 4) * 4 * n_tiles;
+        if (up) hipLaunchKernelGGL((grouped_big_kernel<true>), dim3(blocks), dim3(256), 65536, s, a, n_tiles);
+        else hipLaunchKernelGGL((grouped_big_kernel<false>), dim3(blocks), dim3(256), 65536, s, a, n_tiles);
+    } else if (dtype == TRIMKV_BF16) {
+        if (up) hipLaunchKernelGGL((grouped_skinny_kernel<true>), grid, dim3(256), 0, s, a);
+        else hipLaunchKernelGGL((grouped_skinny_kernel<false>), grid, dim3(256), 0, s, a);
+    } else {
+        if (up) hipLaunchKernelGGL((grouped_simple_kernel<float, true>), grid, dim3(256), 0, s, a);
+        else hipLaunchKernelGGL((grouped_simple_kernel<float, false>), grid, dim3(256), 0, s, a);
+    }
     return launch_status(fn);
 }

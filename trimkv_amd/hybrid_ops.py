@@ -185,9 +185,11 @@ def mlstm(proj: torch.Tensor, offsets: Sequence[int], gates: torch.Tensor, i_bia
     qo, ko, vo, go = offsets
     o = torch.empty(T, s.heads, s.vdim, dtype=torch.float32, device=proj.device)
     out = torch.empty(T, s.heads * s.vdim, dtype=proj.dtype, device=proj.device)
+    need = lib.trimkv_mlstm_workspace(batch.batch, batch.max_len, s.heads, s.dim, s.vdim, code)
+    ws = torch.empty(need, dtype=torch.float32, device=proj.device) if need else None
     _check(lib.trimkv_mlstm(proj.data_ptr(), proj.stride(0), qo, ko, vo, gates.data_ptr(), i_bias.data_ptr(), f_bias.data_ptr(), s.gate_cap,
                             state["S"].data_ptr(), state["nm"].data_ptr(), batch.cu_dev.data_ptr(), batch.slots_dev.data_ptr(), batch.seen_dev.data_ptr(),
-                            o.data_ptr(), batch.batch, batch.max_len, s.heads, s.dim, s.vdim, batch.num_slots, s.dim ** -0.5, code, st), "trimkv_mlstm")
+                            o.data_ptr(), batch.batch, batch.max_len, s.heads, s.dim, s.vdim, batch.num_slots, s.dim ** -0.5, _lib.ptr(ws), code, st), "trimkv_mlstm")
     _check(lib.trimkv_head_norm_gate(o.data_ptr(), proj.data_ptr() + go * proj.element_size(), proj.stride(0), head_norm.data_ptr(), out.data_ptr(),
                                      T, s.heads, s.vdim, eps, code, st), "trimkv_head_norm_gate")
     return out
@@ -218,7 +220,7 @@ def experts(x: torch.Tensor, ids: torch.Tensor, up: torch.Tensor, down: torch.Te
     E, ffp, wp = up.shape
     T, top = ids.shape
     M, dev, lib, st, code = T * top, x.device, _lib.load_hybrid(), _lib.current_stream(x.device), _lib.dtype_code(up.dtype)
-    tile = 16
+    tile = 128 if up.dtype == torch.bfloat16 and M >= 32 * E else 16      # a few rows per expert: stream the weights past them
     most = M if M < E else (M - E) // tile + E
     order = torch.empty(M, dtype=torch.int32, device=dev)
     offsets = torch.empty(E + 1, dtype=torch.int32, device=dev)
