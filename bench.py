@@ -626,6 +626,226 @@ def shell_main(args):
     print(json.dumps(out))
 
 
+HYBRID_SIZES = {
+    # width, attention heads / KV heads (head_dim 128), window, kept first tokens, mLSTM heads (128 x 256), experts, chosen, expert ff
+    # (the chosen experts' two matrices together hold as many weights as the shell's three MLP matrices of 3 x width)
+    "8b": dict(W=4096, Hq=32, Hkv=8, window=4032, keep=64, mh=16, E=32, top=4, ff=4608, B=64),
+    "1.7b": dict(W=2048, Hq=16, Hkv=8, window=1984, keep=64, mh=8, E=32, top=4, ff=2304, B=16),
+}
+
+
+def hybrid_main(args):
+    """Secondary workload (--hybrid): the Fusitar decoder (two windowed-attention and two mLSTM layers, routed experts, random
+    bf16 weights) beside the thin Qwen3 decoder at equal width, head counts, attended rows and weights read per token: prompt
+    and decode throughput of both, and the time of every kernel of the new design against its roofline next to the like
+    kernel of the shell.  Timings of the two decoders alternate."""
+    import torch
+    import torch.nn.functional as F
+    from trimkv_amd import _lib, hybrid_ops as ops, TrimKVCache, get_attention_interface
+    from trimkv_amd.fusitar import FusitarConfig, FusitarForCausalLM
+    from trimkv_amd.graphed import GraphedDecoder
+    from trimkv_amd.qwen3 import TrimKVQwen3Config, TrimKVQwen3ForCausalLM
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    gen = torch.Generator(device=dev).manual_seed(0)
+    MFMA, HBM = 2500e12, 8e12
+
+    def timed(fn, reps, warm=2):
+        for i in range(warm):
+            fn(i)
+        torch.cuda.synchronize()
+        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        e0.record()
+        for i in range(reps):
+            fn(i)
+        e1.record()
+        torch.cuda.synchronize()
+        return e0.elapsed_time(e1) * 1e-3 / reps
+
+    results = {}
+    for name in ([args.hybrid_size] if args.hybrid_size else list(HYBRID_SIZES)):
+        z = HYBRID_SIZES[name]
+        W, B, L, V = z["W"], args.batch or z["B"], 4, 1024
+        M = z["window"] + z["keep"]
+        moe = {"kind": "moe", "expert": {"ff": z["ff"]}, "router": {"experts": z["E"], "top": z["top"], "groups": {"count": 4, "keep": 2}}}
+        att = {"type": "attention", "mlp": moe, "mixer": {"heads": z["Hq"], "kv_heads": z["Hkv"], "dim": D, "vdim": D, "scale": D ** -0.5,
+                                                         "mask": {"size": z["window"], "keep_first": z["keep"]}}}
+        rec = {"type": "mlstm", "mlp": moe, "mixer": {"heads": z["mh"], "dim": 128, "vdim": 256, "gate_cap": 15.0}}
+        cfg = FusitarConfig.from_dict({"vocab": V, "width": W, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6}, "layers": [rec, att, rec, att]})
+        torch.manual_seed(0)
+        with torch.device(dev):
+            model = FusitarForCausalLM(cfg)
+        model.randomize()
+        for i in (0, 2):
+            model.model.layers[i].mix.f_bias.fill_(4.0)
+        qcfg = TrimKVQwen3Config(vocab_size=V, hidden_size=W, intermediate_size=3 * W, num_hidden_layers=L, num_attention_heads=z["Hq"], num_key_value_heads=z["Hkv"],
+                                 head_dim=D, retention_gate="rg", retention_gate_bias_init=3.0, memory_size=M, buffer_size=128)
+        torch.set_default_dtype(torch.bfloat16)
+        with torch.device(dev):
+            shell = TrimKVQwen3ForCausalLM(qcfg)
+        torch.set_default_dtype(torch.float32)
+        shell.eval()
+        ids = lambda b, s: torch.randint(0, V, (b, s), generator=gen, device=dev)
+        r = results[name] = {"layers": L, "width": W, "prefill": {}, "decode": {}}
+
+        with torch.no_grad():
+            for b, s in ((1, 8192), (4, 2048)):
+                x = ids(b, s)
+
+                def prompt_new(i):
+                    cache = model.new_cache(b)
+                    model(x, past_key_values=cache, logits_to_keep=1)
+
+                both = []
+                for _ in range(2):
+                    both.append((timed(prompt_new, 3), timed(lambda i: shell(x, logits_to_keep=1), 3)))
+                new_s, old_s = (min(t) for t in zip(*both))
+                r["prefill"][f"{b} x {s}"] = {"fusitar_tokens_per_s": round(b * s / new_s), "qwen3_shell_tokens_per_s": round(b * s / old_s),
+                                              "fusitar_ms": round(new_s * 1e3, 3), "qwen3_shell_ms": round(old_s * 1e3, 3)}
+            torch.cuda.empty_cache()
+            for b in sorted({1, B}):
+                cache, old = model.new_cache(b), None
+                x = ids(b, M)
+                step = max(1, 16384 // b)
+                for s0 in range(0, M, step):
+                    model(x[:, s0:s0 + step], past_key_values=cache, logits_to_keep=1)
+                    old = shell(x[:, s0:s0 + step], past_key_values=old, logits_to_keep=1).past_key_values
+                nxt = ids(b, 1)
+                n = 12
+                t_eager = timed(lambda i: model(nxt, past_key_values=cache, logits_to_keep=1), n)
+                o_eager = timed(lambda i: shell(nxt, past_key_values=old, logits_to_keep=1), n)
+                dec, odec = GraphedDecoder(model, cache, logits_to_keep=1), GraphedDecoder(shell, old, logits_to_keep=1)
+                t_graph = timed(lambda i: dec(input_ids=nxt), n, 3)
+                o_graph = timed(lambda i: odec(input_ids=nxt), n, 3)
+                t_graph, o_graph = min(t_graph, timed(lambda i: dec(input_ids=nxt), n)), min(o_graph, timed(lambda i: odec(input_ids=nxt), n))
+                dec.close()
+                odec.close()
+                r["decode"][f"batch {b}"] = {"fusitar_tokens_per_s": round(b / min(t_eager, t_graph)), "qwen3_shell_tokens_per_s": round(b / min(o_eager, o_graph)),
+                                             "fusitar_ms": {"eager": round(t_eager * 1e3, 3), "graph": round(t_graph * 1e3, 3)},
+                                             "qwen3_shell_ms": {"eager": round(o_eager * 1e3, 3), "graph": round(o_graph * 1e3, 3)}}
+                if b != B:
+                    del cache, old, dec, odec
+            del old, odec
+            torch.cuda.empty_cache()
+
+            # ---- kernel by kernel ----------------------------------------------------------------------
+            T = 8192
+            k = r["kernels"] = {}
+            l_att, l_rec = [model.model.layers[i] for i in (1, 3)], [model.model.layers[i] for i in (0, 2)]
+            xw = ops.padded(W)
+            big = torch.randn(T, xw, generator=gen, device=dev)
+            bigh = big.to(torch.bfloat16)
+
+            def put(key, sec, flops=0.0, nbytes=0.0, note=None):
+                bound = max(flops / MFMA, nbytes / HBM)
+                k[key] = {"us": round(sec * 1e6, 1), "bound": "mfma" if flops / MFMA >= nbytes / HBM else "hbm", "frac_of_roofline": round(bound / sec, 3)}
+                if note:
+                    k[key]["note"] = note
+
+            pcache = model.new_cache(1)
+            (slot,) = pcache.allocate(1)
+            pb = pcache.batch([T], [slot])
+            proj = torch.randn(T, l_att[0].mix.qkvg.weight.shape[0], generator=gen, device=dev).to(torch.bfloat16)
+            spec, starts = l_att[0].mix.spec, l_att[0].mix.qkvg.starts("q", "k", "v", "g")
+            lib, st = _lib.load_hybrid(), _lib.current_stream(dev)
+            q = torch.randn(T, spec.heads, D, generator=gen, device=dev).to(torch.bfloat16)
+            kk = torch.randn(T, spec.kv_heads, D, generator=gen, device=dev).to(torch.bfloat16)
+            vv = torch.randn(T, spec.kv_heads, D, generator=gen, device=dev).to(torch.bfloat16)
+            out = torch.empty(T, spec.heads * D, dtype=torch.bfloat16, device=dev)
+            ring = pcache.layers_state[1]
+            shape = (spec.heads, spec.kv_heads, D, D, D, D, spec.keep_first, spec.window)
+            gate = proj.data_ptr() + starts[3] * 2
+
+            def window_prefill(i):
+                _lib.check_hybrid(lib.trimkv_window_prefill(q.data_ptr(), kk.data_ptr(), vv.data_ptr(), ring["k"].data_ptr(), ring["v"].data_ptr(), pb.cu_dev.data_ptr(),
+                                                            pb.slots_dev.data_ptr(), pb.seen_dev.data_ptr(), gate, proj.stride(0), out.data_ptr(), 1, T, *shape, spec.scale, _lib.BF16, st), "window")
+            seen_pairs = sum(min(t + 1, spec.window + min(spec.keep_first, max(0, t + 1 - spec.window))) for t in range(T))
+            put("window_prefill", timed(window_prefill, 10), flops=4.0 * D * spec.heads * seen_pairs, note=f"{T} tokens")
+            attn = get_attention_interface("trimkv_hip")
+
+            class Mod:
+                training, num_key_value_groups = False, z["Hq"] // z["Hkv"]
+            oc = TrimKVCache()
+            lb = torch.zeros(1, z["Hkv"], T, device=dev)
+            K_, V_, _, _, kw = oc.update(kk.view(1, T, -1, D).transpose(1, 2), vv.view(1, T, -1, D).transpose(1, 2), lb, torch.arange(T, device=dev), 0)
+            q4 = q.view(1, T, -1, D).transpose(1, 2)
+            put("shell: prefill attention", timed(lambda i: attn(Mod(), q4, K_, V_, None, scaling=D ** -0.5, flash_attn_kwargs=kw), 10),
+                flops=4.0 * D * spec.heads * T * (T + 1) / 2, note=f"{T} tokens, causal")
+            del oc, K_, V_
+            put("qkv_norm (prompt)", timed(lambda i: _lib.check_hybrid(lib.trimkv_qkv_norm(
+                proj.data_ptr(), proj.stride(0), *starts[:3], l_att[0].mix.q_norm.data_ptr(), l_att[0].mix.k_norm.data_ptr(), 1e-6, spec.heads, spec.kv_heads, D, D, D, D,
+                q.data_ptr(), kk.data_ptr(), vv.data_ptr(), None, None, 0, 0, T, _lib.BF16, st), "qkv"), 10), nbytes=2.0 * 2 * T * (spec.heads + 2 * spec.kv_heads) * D)
+            ms = l_rec[0].mix
+            mproj = torch.randn(T, ms.qkvg.weight.shape[0], generator=gen, device=dev).to(torch.bfloat16)
+            gates = torch.randn(T, 2 * ms.spec.heads, generator=gen, device=dev)
+            mst = ms.qkvg.starts("q", "k", "v", "g")
+            f_new = lambda p, g, cache, layer, batch: ops.mlstm(p, mst, g, ms.i_bias, ms.f_bias, ms.head_norm, 1e-6, ms.spec, cache.layers_state[layer], batch)
+            h_, d_, dv_ = ms.spec.heads, ms.spec.dim, ms.spec.vdim
+            put("mlstm (prompt, with head norm)", timed(lambda i: f_new(mproj, gates, pcache, 0, pb), 10), flops=T * h_ * (2.0 * 64 * (d_ + dv_) + 4.0 * d_ * dv_),
+                nbytes=T * h_ * 2.0 * (2 * d_ + 3 * dv_), note=f"{T} tokens, chunks of 64")
+            moe_l = l_att[0].mlp
+            ids_, wts = ops.route(ops.linear_f32(big, moe_l.router), moe_l.correction, moe_l.spec)
+            put("router product (prompt)", timed(lambda i: ops.linear_f32(big, moe_l.router), 10), nbytes=4.0 * T * W)
+            put("route (prompt)", timed(lambda i: ops.route(wts.new_zeros(T, z["E"]), moe_l.correction, moe_l.spec), 10), nbytes=4.0 * T * (z["E"] + 2 * z["top"]))
+            put("experts (prompt: plan, up, down)", timed(lambda i: ops.experts(bigh, ids_, l_att[i % 2].mlp.up, l_att[i % 2].mlp.down, W), 6), flops=4.0 * T * z["top"] * W * z["ff"])
+            wg = torch.randn(3 * W, W, generator=gen, device=dev).to(torch.bfloat16)
+            put("shell: vendor GEMM (prompt)", timed(lambda i: F.linear(bigh[:, :W], wg), 10), flops=2.0 * T * 3 * W * W)
+            y = ops.experts(bigh, ids_, moe_l.up, moe_l.down, W)
+            put("residual_norm over experts (prompt)", timed(lambda i: ops.residual_norm(big, bigh, y, l_att[0].norm2, 1e-6, wts), 10), nbytes=T * W * (2.0 * z["top"] + 4 + 4 + 2))
+            y1 = y[:T].contiguous()
+            put("residual_norm (prompt)", timed(lambda i: ops.residual_norm(big, bigh, y1, l_att[0].norm1, 1e-6), 10), nbytes=T * W * (2.0 + 4 + 4 + 2))
+            from trimkv_amd import decoder_ops
+            nw = torch.ones(W, device=dev, dtype=torch.bfloat16)
+            put("shell: rmsnorm with residual (prompt)", timed(lambda i: decoder_ops.rmsnorm(y1, nw, 1e-6, y1), 10), nbytes=T * W * 2.0 * 4)
+            del proj, q, kk, vv, out, mproj, y, y1, pcache, wg
+            torch.cuda.empty_cache()
+            # decode, batch B, on the cache of the steps above (window full); layers alternate so that nothing stays in a cache
+            db = cache.batch([1] * B)
+            aproj = torch.randn(B, l_att[0].mix.qkvg.weight.shape[0], generator=gen, device=dev).to(torch.bfloat16)
+            mproj = torch.randn(B, ms.qkvg.weight.shape[0], generator=gen, device=dev).to(torch.bfloat16)
+            am = l_att[0].mix
+            qd = torch.randn(B, spec.heads, D, generator=gen, device=dev).to(torch.bfloat16)
+            od = torch.empty(B, spec.heads * D, dtype=torch.bfloat16, device=dev)
+            splits = lib.trimkv_window_decode_splits(B, spec.kv_heads, spec.rows)
+            ws = torch.empty(B * spec.heads * splits * (D + 2), device=dev)
+
+            def window_decode(i):
+                rg = cache.layers_state[1 + 2 * (i % 2)]
+                _lib.check_hybrid(lib.trimkv_window_decode(qd.data_ptr(), rg["k"].data_ptr(), rg["v"].data_ptr(), db.slots_dev.data_ptr(), db.seen_dev.data_ptr(), aproj.data_ptr() + starts[3] * 2,
+                                                           aproj.stride(0), od.data_ptr(), B, *shape, spec.scale, splits, ws.data_ptr(), _lib.BF16, st), "window")
+            put(f"window_decode (batch {B})", timed(window_decode, 20), nbytes=2.0 * 2 * B * spec.kv_heads * spec.rows * D)
+            oc = TrimKVCache()
+            for l in range(2):
+                kd = torch.randn(B, z["Hkv"], M, D, generator=gen, device=dev, dtype=torch.bfloat16)
+                oc.update(kd, kd, torch.zeros(B, z["Hkv"], M, device=dev), torch.arange(M, device=dev), l)
+            del kd
+            q4 = qd.view(B, spec.heads, 1, D)
+            views = [(oc.key_cache[l], oc.value_cache[l], {"seg_len": oc._slabs[l].seg_len, "max_len": M, "seg_cap": oc._slabs[l].cap}) for l in range(2)]
+            put(f"shell: decode attention (batch {B})", timed(lambda i: attn(Mod(), q4, views[i % 2][0], views[i % 2][1], None, scaling=D ** -0.5, flash_attn_kwargs=views[i % 2][2]), 20),
+                nbytes=2.0 * 2 * B * spec.kv_heads * M * D)
+            del oc, views
+            gd = torch.randn(B, 2 * h_, generator=gen, device=dev)
+            put(f"mlstm (decode, batch {B}, with head norm)", timed(lambda i: f_new(mproj, gd, cache, 2 * (i % 2), db), 20), nbytes=2.0 * 4 * B * h_ * d_ * dv_)
+            xd, xdh = big[:B].contiguous(), bigh[:B].contiguous()
+            ids_, wts = ops.route(ops.linear_f32(xd, moe_l.router), moe_l.correction, moe_l.spec)
+            used = len(set(ids_.flatten().tolist()))
+            put(f"experts (decode, batch {B}: plan, up, down)", timed(lambda i: ops.experts(xdh, ids_, l_att[i % 2].mlp.up, l_att[i % 2].mlp.down, W), 20), nbytes=2.0 * used * 2 * W * z["ff"])
+            wd = [torch.randn(3 * W, W, generator=gen, device=dev).to(torch.bfloat16) for _ in range(4)]
+            put(f"shell: vendor GEMM (decode, batch {B})", timed(lambda i: F.linear(xdh[:, :W], wd[i % 4]), 20), nbytes=2.0 * 3 * W * W)
+            put(f"router product (decode, batch {B})", timed(lambda i: ops.linear_f32(xd, moe_l.router), 20), nbytes=4.0 * B * W + 2.0 * z["E"] * W)
+            put(f"residual_norm (decode, batch {B})", timed(lambda i: ops.residual_norm(xd, xdh, xdh, l_att[0].norm1, 1e-6), 20), nbytes=B * W * (2.0 + 4 + 4 + 2))
+        del model, shell, cache, dec
+        torch.cuda.empty_cache()
+    first = next(iter(results.values()))
+    dec = first["decode"][max(first["decode"], key=lambda s: int(s.split()[1]))]
+    ms = min(dec["fusitar_ms"].values())
+    print(json.dumps({
+        "metric": "decode tokens/s of the Fusitar decoder (4 layers, random weights) beside the thin Qwen3 decoder", "value": dec["fusitar_tokens_per_s"], "unit": "tokens/s",
+        "n_gpus": 1, "steps": 12, "warmup": 2, "ms_per_step": ms, "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "4 layers (mLSTM, windowed attention, twice), routed experts, sizes per entry of `results`", "note": "secondary workload; the headline metric is the default run"},
+        "results": results}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -665,6 +885,10 @@ def main():
     ap.add_argument("--prefill", action="store_true",
                     help="secondary workload: chunked prompt processing at config 5's shape (4096-token chunks); "
                          "with it --steps/--warmup count chunks (defaults 6/2)")
+    ap.add_argument("--hybrid", action="store_true",
+                    help="secondary workload: prompt and decode throughput of the Fusitar decoder beside the thin Qwen3 decoder at equal size, "
+                         "and its kernels against their rooflines")
+    ap.add_argument("--hybrid-size", choices=sorted(HYBRID_SIZES), help="--hybrid only: one of the sizes (default: all)")
     args = ap.parse_args()
     if args.event_every < 0:
         args.event_every = max(8, args.steps // 16)
@@ -677,6 +901,8 @@ def main():
         if args.steps == 1024 and args.warmup == 128:
             args.steps, args.warmup = 6, 2
         return prefill_main(args)
+    if args.hybrid:
+        return hybrid_main(args)
     if args.shell:
         if args.steps == 1024 and args.warmup == 128:
             args.steps, args.warmup = 12, 3

@@ -93,8 +93,10 @@ int trimkv_moe_route(const float* logits, const float* correction, int32_t* ids,
  * (expert, first row) of every run of up to `tile` rows; most = rows < experts ? rows : (rows - experts) / tile + experts. */
 int trimkv_moe_plan(const int32_t* ids, int rows, int experts, int tile, int32_t* order, int32_t* offsets, int32_t* tiles, void* stream);
 
-/* One product per expert: w [experts][n_padded][k_padded], zeros in the padding (multiples of 64).  up: y[i] =
- * relu(w x[order[i] / top])^2; else y[order[i]] = w x[i].  `tile` as in the plan: 16 or (bf16) 128. */
+/* One product per expert.  w: n and k padded with zeros to multiples of 64, stored in blocks of 32 outputs x 16 k as the matrix
+ * cores take them, [experts][n_padded / 32][k_padded / 16][2][32][8]: first k 0..7 of the block's 32 outputs, then k 8..15.
+ * up: y[i] = relu(w x[order[i] / top])^2; else y[order[i]] = w x[i].  x rows hold k_padded elements.  `tile` as in the plan:
+ * 16 in fp32, in bf16 32 (a few rows per expert) or 256. */
 int trimkv_moe_gemm(const void* x, int64_t x_stride, const void* w, void* y, int64_t y_stride, const int32_t* order, const int32_t* offsets,
                     const int32_t* tiles, int rows, int experts, int tile, int top, int n, int n_padded, int k_padded, int up, int dtype, void* stream);
 

@@ -74,9 +74,8 @@ def run_window(spec, dtype, seqs, cuts, stand_out=()):
     offs = [0, sizes[0], sizes[0] + sizes[1], sum(sizes[:3])]
     rows = [rnd(n, sum(sizes), seed=20 + i) for i, n in enumerate(seqs)]
     for b, qi, kj in stand_out:
-        # one direction per pair: the KV head's own pattern repeated over its query heads, flipped by the norm weights' sign
-        u = rnd(G, D, seed=1000 + kj) * 6.0
-        rows[b][kj, offs[1]:offs[2]] = (u / kw.view(G, D)).reshape(-1) if False else u.reshape(-1)
+        u = rnd(G, D, seed=1000 + kj) * 6.0          # one direction per KV head, shared by its query heads
+        rows[b][kj, offs[1]:offs[2]] = u.reshape(-1)
         rows[b][qi, :offs[1]] = u.repeat_interleave(H // G, dim=0).reshape(-1)
     rows = [r.to(dtype) for r in rows]
     want = []
@@ -264,6 +263,6 @@ def test_experts(dtype, T, E, top, ff, width):
     ids = torch.stack([torch.randperm(E, generator=gen)[:top] for _ in range(T)]).int()
     if E > 4:
         ids[ids == 2] = 0 if top == 1 else ids[ids == 2]          # an expert nobody asks for
-    y = ops.experts(x.to(DEV), ids.to(DEV), up.to(DEV), down.to(DEV), width).view(T, top, width)
+    y = ops.experts(x.to(DEV), ids.to(DEV), ops.pack_matrix(up).contiguous().to(DEV), ops.pack_matrix(down).contiguous().to(DEV), width).view(T, top, width)
     want = torch.stack([torch.stack([ref.expert(x[t].double()[:width], up[e].double()[:ff, :width], down[e].double()[:width, :ff]) for e in ids[t].tolist()]) for t in range(T)])
     close(y, want, 2e-6 if dtype == torch.float32 else 1.2e-2)

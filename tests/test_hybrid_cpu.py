@@ -12,6 +12,7 @@ from safetensors.torch import save_file
 
 from oracle import hybrid_ref as ref
 from trimkv_amd import _lib, registry
+from trimkv_amd.hybrid_ops import pack_matrix, unpack_matrix
 from trimkv_amd.fusitar import FusitarConfig, FusitarForCausalLM
 from tests.hybrid_util import attention, config, mlstm, moe, weights
 
@@ -43,7 +44,7 @@ def test_bad_arguments_are_refused_without_a_launch():
     assert lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, 4, 2, 16, 16, 16, 16, 1, 4, 1.0, 3, None, _lib.BF16, None) == -5
     assert lib.trimkv_moe_route(one, one, one, one, 1, 8, 5, 2, 1, None) == -2          # one open group of four cannot give five
     assert lib.trimkv_moe_route(one, one, one, one, 1, 9, 2, 2, 1, None) == -2
-    assert lib.trimkv_moe_gemm(one, 64, one, one, 64, one, one, one, 4, 2, 32, 1, 64, 64, 64, 1, _lib.BF16, None) == -2
+    assert lib.trimkv_moe_gemm(one, 64, one, one, 64, one, one, one, 4, 2, 16, 1, 64, 64, 64, 1, _lib.BF16, None) == -2
     assert lib.trimkv_mlstm(one, 64, 0, 8, 16, one, one, one, 1.0, one, one, one, one, one, one, 1, 1, 1, 513, 8, 1, 1.0, None, _lib.F32, None) == -6
     assert lib.trimkv_window_decode_splits(64, 8, 4096) >= 1 and lib.trimkv_window_decode_splits(1, 1, 64) == 1
     assert lib.trimkv_mlstm_workspace(1, 1, 4, 64, 64, _lib.BF16) == 0
@@ -76,9 +77,13 @@ def test_loading_fills_every_parameter_and_refuses_what_does_not_fit(tmp_path):
     save_file(w, str(tmp_path / "model.safetensors"))
     model = registry.from_pretrained(str(tmp_path), torch_dtype=torch.float32)
     for name, t in model.tensors().items():
-        assert torch.equal(t, w[name].float()), name
+        assert torch.equal(t.value() if hasattr(t, "value") else t, w[name].float()), name
     # padding stays zero: kernels read it
-    assert not model.model.layers[0].mlp.up[:, 40:].any() and not model.model.layers[0].mlp.down[:, :, 40:].any()
+    up, down = (unpack_matrix(m.data) for m in (model.model.layers[0].mlp.up, model.model.layers[0].mlp.down))
+    assert up.shape == (6, 64, 128) and not up[:, 40:].any() and not up[:, :, 72:].any() and not down[:, 72:].any() and not down[:, :, 40:].any()
+    # block (n / 32, k / 16): k 0..7 of its 32 outputs, then k 8..15
+    m = torch.arange(64 * 128).view(64, 128)
+    assert pack_matrix(m)[1, 3, 1, 5].tolist() == m[37, 56:64].tolist() and torch.equal(unpack_matrix(pack_matrix(m)), m)
     for change in (lambda d: d.pop("l1.mix.f.b"), lambda d: d.update(extra=torch.zeros(1)), lambda d: d.update({"l0.norm1": torch.zeros(71)})):
         bad = dict(w)
         change(bad)

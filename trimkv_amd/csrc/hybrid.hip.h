@@ -92,6 +92,13 @@ __device__ __forceinline__ void load_to_lds16(const void* src, uint32_t lds_addr
                  : "=&s"(saved) : "v"(src), "s"(lds_addr) : "memory");
 }
 
+// the same from a wavefront-uniform base and a per-lane byte offset
+__device__ __forceinline__ void load_to_lds16_at(const char* base, uint32_t offset, uint32_t lds_addr) {
+    uint32_t saved;
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0"
+                 : "=&s"(saved) : "v"(offset), "s"(base), "s"(lds_addr) : "memory");
+}
+
 // The slot of a token in a window ring: the first `keep` positions own their slots, later ones take turns on `size` slots.
 __device__ __forceinline__ int ring_slot(int pos, int keep, int size) { return pos < keep ? pos : keep + (pos - keep) % size; }
 // The position a ring slot holds after `total` tokens (total > slot): the newest one that maps to it.

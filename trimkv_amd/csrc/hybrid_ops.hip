@@ -91,27 +91,52 @@ struct ResidualNormArgs {
     const void* y; int64_t y_stride; const float* y_weight; int top;
     float* x; const float* w; void* xh; int width, xs; float eps;
 };
-template <typename T, bool VEC>
+// NV > 0: rows of up to 1024 NV elements, four at a time, held in registers; everything is requested before the reduction.
+template <typename T, int NV>
 __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) {
-    extern __shared__ float row[];     // width floats: y of this token, summed over its experts
+    extern __shared__ float row[];     // NV = 0: width floats, y of this token summed over its experts
     __shared__ float part[4];
     const int64_t t = blockIdx.x;
     const int tid = threadIdx.x;
     const T* y = (const T*)a.y + t * a.top * a.y_stride;
+    float* xr = a.x + t * a.xs;
+    T* hr = (T*)a.xh + t * a.xs;
     float ss = 0.0f;
-    if constexpr (VEC) {
-        for (int i = tid * 4; i < a.width; i += 1024) {
-            float4 s;
-            if (a.y_weight) {
-                s = make_float4(0.f, 0.f, 0.f, 0.f);
-                for (int j = 0; j < a.top; ++j) {
-                    const float wt = a.y_weight[t * a.top + j];
-                    const float4 f = ld4(y + j * a.y_stride + i);
-                    s.x += wt * f.x; s.y += wt * f.y; s.z += wt * f.z; s.w += wt * f.w;
+    if constexpr (NV > 0) {
+        float4 s[NV], f[NV], w[NV];
+#pragma unroll
+        for (int v = 0; v < NV; ++v) {
+            const int i = (v * 256 + tid) * 4;
+            s[v] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (i < a.width) {
+                f[v] = *(const float4*)(xr + i);
+                w[v] = *(const float4*)(a.w + i);
+                if (!a.y_weight) s[v] = ld4(y + i);
+            }
+        }
+        if (a.y_weight)
+            for (int j = 0; j < a.top; ++j) {
+                const float wt = a.y_weight[t * a.top + j];
+#pragma unroll
+                for (int v = 0; v < NV; ++v) {
+                    const int i = (v * 256 + tid) * 4;
+                    if (i < a.width) {
+                        const float4 e = ld4(y + j * a.y_stride + i);
+                        s[v].x += wt * e.x; s[v].y += wt * e.y; s[v].z += wt * e.z; s[v].w += wt * e.w;
+                    }
                 }
-            } else s = ld4(y + i);
-            *(float4*)(row + i) = s;
-            ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
+            }
+#pragma unroll
+        for (int v = 0; v < NV; ++v) ss += s[v].x * s[v].x + s[v].y * s[v].y + s[v].z * s[v].z + s[v].w * s[v].w;
+        const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+#pragma unroll
+        for (int v = 0; v < NV; ++v) {
+            const int i = (v * 256 + tid) * 4;
+            if (i < a.width) {
+                f[v].x += s[v].x * inv * w[v].x; f[v].y += s[v].y * inv * w[v].y; f[v].z += s[v].z * inv * w[v].z; f[v].w += s[v].w * inv * w[v].w;
+                *(float4*)(xr + i) = f[v];
+                if (a.xh) st4(hr + i, f[v]);
+            }
         }
     } else {
         for (int i = tid; i < a.width; i += 256) {
@@ -121,20 +146,8 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
             row[i] = s;
             ss += s * s;
         }
-    }
-    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
-    float* xr = a.x + t * a.xs;
-    T* hr = (T*)a.xh + t * a.xs;
-    if constexpr (VEC) {
-        for (int i = tid * 4; i < a.width; i += 1024) {     // a thread re-reads what it wrote itself
-            const float4 s = *(const float4*)(row + i), w = *(const float4*)(a.w + i);
-            float4 f = *(const float4*)(xr + i);
-            f.x += s.x * inv * w.x; f.y += s.y * inv * w.y; f.z += s.z * inv * w.z; f.w += s.w * inv * w.w;
-            *(float4*)(xr + i) = f;
-            if (a.xh) st4(hr + i, f);
-        }
-    } else {
-        for (int i = tid; i < a.width; i += 256) {
+        const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+        for (int i = tid; i < a.width; i += 256) {      // a thread re-reads what it wrote itself
             const float f = xr[i] + row[i] * inv * a.w[i];
             xr[i] = f;
             if (a.xh) st(hr + i, f);
@@ -162,6 +175,74 @@ struct QkvNormArgs {
     const int32_t* slots; const int32_t* seen;       // both given: k and v rows go into the rings k, v [slot][G][cap][padded dim]
     int keep, size;
 };
+// rows of heads without padding and multiples of 8 apart: eight elements at a time
+struct Eight { float f[8]; };
+__device__ __forceinline__ Eight ld8(const bf16_t* p) {
+    const hy_u32x4 r = *(const hy_u32x4*)p;
+    Eight e;
+#pragma unroll
+    for (int x = 0; x < 4; ++x) { e.f[2 * x] = __uint_as_float(r[x] << 16); e.f[2 * x + 1] = __uint_as_float(r[x] & 0xffff0000u); }
+    return e;
+}
+__device__ __forceinline__ Eight ld8(const float* p) {
+    const float4 a = *(const float4*)p, b = *(const float4*)(p + 4);
+    return {{a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w}};
+}
+__device__ __forceinline__ void st8(bf16_t* p, Eight e) { *(hy_u32x4*)p = hy_u32x4{pack2(e.f[0], e.f[1]), pack2(e.f[2], e.f[3]), pack2(e.f[4], e.f[5]), pack2(e.f[6], e.f[7])}; }
+__device__ __forceinline__ void st8(float* p, Eight e) { *(float4*)p = make_float4(e.f[0], e.f[1], e.f[2], e.f[3]); *(float4*)(p + 4) = make_float4(e.f[4], e.f[5], e.f[6], e.f[7]); }
+
+template <typename T>
+__global__ __launch_bounds__(256) void qkv_norm_vec_kernel(QkvNormArgs a) {
+    __shared__ float part[4];
+    const int64_t t = blockIdx.x;
+    const int tid = threadIdx.x, kind = blockIdx.y;
+    const T* row = (const T*)a.p + t * a.p_stride;
+    const T* src = row + (kind ? a.k_off : a.q_off);
+    const float* wt = kind ? a.kw : a.qw;
+    const int n = (kind ? a.G : a.H) * a.D;
+    constexpr int HOLD = 2;                               // held in registers between the two passes; longer rows are read again
+    Eight held[HOLD];
+    float ss = 0.0f;
+#pragma unroll
+    for (int v = 0; v < HOLD; ++v) {
+        const int i = (v * 256 + tid) * 8;
+        if (i < n) {
+            held[v] = ld8(src + i);
+#pragma unroll
+            for (int x = 0; x < 8; ++x) ss += held[v].f[x] * held[v].f[x];
+        }
+    }
+    for (int i = (HOLD * 256 + tid) * 8; i < n; i += 2048) {
+        const Eight e = ld8(src + i);
+#pragma unroll
+        for (int x = 0; x < 8; ++x) ss += e.f[x] * e.f[x];
+    }
+    int64_t kstep = a.D, vstep = a.Dv, k0 = t * a.G * a.D, v0 = t * a.G * a.Dv;
+    if (kind && a.slots) {
+        const int slot = a.slots[t], cap = a.keep + a.size, r = ring_slot(a.seen[2 * slot], a.keep, a.size);
+        kstep = (int64_t)cap * a.D; vstep = (int64_t)cap * a.Dv;
+        k0 = (int64_t)slot * a.G * kstep + (int64_t)r * a.D; v0 = (int64_t)slot * a.G * vstep + (int64_t)r * a.Dv;
+    }
+    if (kind)
+        for (int i = tid * 8; i < a.G * a.Dv; i += 2048) {
+            const int g = i / a.Dv;
+            st8((T*)a.v + v0 + g * vstep + (i - g * a.Dv), ld8(row + a.v_off + i));
+        }
+    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)n + a.eps);
+    auto put = [&](int i, Eight e) __attribute__((always_inline)) {
+        const Eight w = ld8(wt + i);
+#pragma unroll
+        for (int x = 0; x < 8; ++x) e.f[x] *= inv * w.f[x];
+        if (!kind) { st8((T*)a.q + t * n + i, e); return; }
+        const int g = i / a.D;
+        st8((T*)a.k + k0 + g * kstep + (i - g * a.D), e);
+    };
+#pragma unroll
+    for (int v = 0; v < HOLD; ++v)
+        if ((v * 256 + tid) * 8 < n) put((v * 256 + tid) * 8, held[v]);
+    for (int i = (HOLD * 256 + tid) * 8; i < n; i += 2048) put(i, ld8(src + i));
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void qkv_norm_kernel(QkvNormArgs a) {
     __shared__ float part[4];
@@ -237,6 +318,35 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* o, con
     for (int i = lane; i < Dv; i += 64) st(out + unit * Dv + i, src[i] * inv * w[h * Dv + i] * sigmoid_f(ld(gr + i)));
 }
 
+// Dv a multiple of 4 up to 256 NV: the row is held in registers
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(const float* o, const T* g, int64_t g_stride, const float* w, T* out, int64_t units, int H, int Dv, float eps) {
+    const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (unit >= units) return;
+    const int64_t t = unit / H;
+    const int h = (int)(unit - t * H), lane = threadIdx.x & 63;
+    float4 s[NV], gt[NV], wt[NV];
+    float ss = 0.0f;
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+        const int i = (v * 64 + lane) * 4;
+        s[v] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (i < Dv) {
+            s[v] = ld4(o + unit * Dv + i);
+            gt[v] = ld4(g + t * g_stride + h * Dv + i);
+            wt[v] = ld4(w + h * Dv + i);
+        }
+        ss += s[v].x * s[v].x + s[v].y * s[v].y + s[v].z * s[v].z + s[v].w * s[v].w;
+    }
+    const float inv = 1.0f / sqrtf(wave_sum_f(ss) / (float)Dv + eps);
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+        const int i = (v * 64 + lane) * 4;
+        if (i < Dv) st4(out + unit * Dv + i, make_float4(s[v].x * inv * wt[v].x * sigmoid_f(gt[v].x), s[v].y * inv * wt[v].y * sigmoid_f(gt[v].y),
+                                                         s[v].z * inv * wt[v].z * sigmoid_f(gt[v].z), s[v].w * inv * wt[v].w * sigmoid_f(gt[v].w)));
+    }
+}
+
 __global__ void advance_kernel(int32_t* seen, const int32_t* slots, const int32_t* cu, int batch) {
     const int b = blockIdx.x * 64 + threadIdx.x;
     if (b >= batch) return;
@@ -296,8 +406,11 @@ extern "C" int trimkv_residual_norm(const void* y, int64_t y_stride, const float
     const bool vec = width % 4 == 0 && x_stride % 4 == 0 && y_stride % 4 == 0 && !((((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)xh)) & 15);
     const size_t lds = (size_t)width * 4;
     HY_BY_DTYPE(dtype, T,
-        if (vec) hipLaunchKernelGGL((residual_norm_kernel<T, true>), dim3(tokens), dim3(256), lds, (hipStream_t)stream, a);
-        else hipLaunchKernelGGL((residual_norm_kernel<T, false>), dim3(tokens), dim3(256), lds, (hipStream_t)stream, a));
+        if (vec && width <= 1024) hipLaunchKernelGGL((residual_norm_kernel<T, 1>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+        else if (vec && width <= 2048) hipLaunchKernelGGL((residual_norm_kernel<T, 2>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+        else if (vec && width <= 4096) hipLaunchKernelGGL((residual_norm_kernel<T, 4>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+        else if (vec && width <= 8192) hipLaunchKernelGGL((residual_norm_kernel<T, 8>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+        else hipLaunchKernelGGL((residual_norm_kernel<T, 0>), dim3(tokens), dim3(256), lds, (hipStream_t)stream, a));
     return launch_status(fn);
 }
 
@@ -319,6 +432,12 @@ extern "C" int trimkv_qkv_norm(const void* proj, int64_t proj_stride, int q_off,
     if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || dim_stride < dim || vdim_stride < vdim || (slots && (window <= 0 || keep_first < 0)))
         return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d heads=%d kv_heads=%d dim=%d vdim=%d", fn, tokens, heads, kv_heads, dim, vdim);
     QkvNormArgs a{proj, proj_stride, q_off, k_off, v_off, q_weight, k_weight, eps, heads, kv_heads, dim, vdim, dim_stride, vdim_stride, q, k, v, slots, seen, keep_first, window};
+    const bool vec = dim_stride == dim && vdim_stride == vdim && dim % 8 == 0 && vdim % 8 == 0 && proj_stride % 8 == 0 && (q_off | k_off | v_off) % 8 == 0 &&
+                     !(((uintptr_t)proj | (uintptr_t)q_weight | (uintptr_t)k_weight | (uintptr_t)q | (uintptr_t)k | (uintptr_t)v) & 15);
+    if (vec) {
+        HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((qkv_norm_vec_kernel<T>), dim3(tokens, 2), dim3(256), 0, (hipStream_t)stream, a));
+        return launch_status(fn);
+    }
     HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((qkv_norm_kernel<T>), dim3(tokens, 2), dim3(256), 0, (hipStream_t)stream, a));
     return launch_status(fn);
 }
@@ -341,6 +460,13 @@ extern "C" int trimkv_head_norm_gate(const float* o, const void* gate, int64_t g
     HY_CHECK_DTYPE(fn, dtype);
     if (tokens <= 0 || heads <= 0 || vdim <= 0) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d heads=%d vdim=%d", fn, tokens, heads, vdim);
     const int64_t units = (int64_t)tokens * heads;
+    if (vdim % 4 == 0 && vdim <= 512 && gate_stride % 4 == 0 && !(((uintptr_t)o | (uintptr_t)gate | (uintptr_t)w | (uintptr_t)out) & 15)) {
+        const dim3 grid((unsigned)((units + 3) / 4));
+        HY_BY_DTYPE(dtype, T,
+            if (vdim <= 256) hipLaunchKernelGGL((head_norm_gate_vec_kernel<T, 1>), grid, dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps);
+            else hipLaunchKernelGGL((head_norm_gate_vec_kernel<T, 2>), grid, dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
+        return launch_status(fn);
+    }
     HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((head_norm_gate_kernel<T>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
     return launch_status(fn);
 }

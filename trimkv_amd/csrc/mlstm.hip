@@ -202,11 +202,16 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
         }
     };
     const float ib = a.ib[h], fb = a.fb[h];
-    auto gates = [&](int c, int buf) __attribute__((always_inline)) {     // one wavefront, lane = token of chunk c
+    float zi = 0.0f, zf = 0.0f;                       // raw gates of the chunk after next, on their way
+    auto fetch_gates = [&](int c) __attribute__((always_inline)) {        // one wavefront, lane = token of chunk c
+        const float* g = a.gates + (int64_t)(t0 + first + min(c * 64 + lane, len - 1)) * 2 * a.H + h;
+        zi = g[0];
+        zf = g[a.H];
+    };
+    auto gates = [&](int c, int buf) __attribute__((always_inline)) {
         const int t = c * 64 + lane;
-        const float* g = a.gates + (int64_t)(t0 + first + min(t, len - 1)) * 2 * a.H + h;
-        const float li = t < len ? log_input_gate(g[0] + ib, a.cap) : -1.0e30f;
-        const float lf = t < len ? log_forget_gate(g[a.H] + fb, a.cap) : 0.0f;
+        const float li = t < len ? log_input_gate(zi + ib, a.cap) : -1.0e30f;
+        const float lf = t < len ? log_forget_gate(zf + fb, a.cap) : 0.0f;
         const float F = wave_scan_add(lf, lane), d = li - F;
         gF[buf * 64 + lane] = F;
         gD[buf * 64 + lane] = d;
@@ -225,12 +230,13 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
     const int nchunks = (len + 63) / 64;
     float fsum = 0.0f;
     request(0, 0);
-    if (w == 3) gates(0, 0);
+    if (w == 3) { fetch_gates(0); gates(0, 0); fetch_gates(1); }
     for (int c = 0; c < nchunks; ++c) {
         const int buf = NB == 2 ? c & 1 : 0, gb = (c & 1) * 64, off = buf * C::BUF;
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        if (c == 0 || NB == 1) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();                              // chunk c and its gates are there; chunk c - 1 is done with
         if (NB == 2 && c + 1 < nchunks) request(c + 1, buf ^ 1);
+        if (w == 3 && c + 1 < nchunks) { gates(c + 1, (c + 1) & 1); fetch_gates(c + 2); }
         const float Mc = fmaxf(m0, gM[gb + 63]);
         hy_f32x16 o[2];
         if (MODE != CHUNK_LOCAL) {
@@ -351,24 +357,6 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                         S[db] = mfma32(kf, __builtin_bit_cast(hy_bf16x8, (hy_u32x4){e0[e], e1[e], e2[e], e3[e]}), S[db]);
                 }
             }
-            if (MODE != CHUNK_LOCAL) {
-#pragma unroll
-                for (int tb = 0; tb < 2; ++tb) {
-                    const int t = tb * 32 + j;
-                    const float M = fmaxf(m0, gM[gb + t]);
-                    const float den = dsum[tb * 32 + j] + (tb ? dsum[64 + j] : 0.0f) + exp_fast(m0 - M) * qn[t];
-                    const float inv = 1.0f / (fmaxf(fabsf(den), exp_fast(-(gF[gb + t] + M))) + 1e-6f);
-                    float* orow = a.o + ((int64_t)(t0 + first + c * 64 + t) * a.H + h) * a.Dv + dv0 + w * 32;
-                    if (c * 64 + t < len) {
-#pragma unroll
-                        for (int x = 0; x < 4; ++x) {
-                            const int d = 8 * x + 4 * hl;           // Dv is a multiple of 8: four columns are in or out together
-                            if (dv0 + w * 32 + d < a.Dv)
-                                *(float4*)(orow + d) = make_float4(o[tb][4 * x] * inv, o[tb][4 * x + 1] * inv, o[tb][4 * x + 2] * inv, o[tb][4 * x + 3] * inv);
-                        }
-                    }
-                }
-            }
         }
         // n: 16 pairs of features per wavefront and pass, four quarters of the tokens side by side
         {
@@ -393,7 +381,27 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                 }
             }
         }
-        if (w == 3 && c + 1 < nchunks) gates(c + 1, (c + 1) & 1);
+        if (NB == 2) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the next chunk, requested a chunk ago: not the stores below
+        if (live) {
+            if (MODE != CHUNK_LOCAL) {
+#pragma unroll
+                for (int tb = 0; tb < 2; ++tb) {
+                    const int t = tb * 32 + j;
+                    const float M = fmaxf(m0, gM[gb + t]);
+                    const float den = dsum[tb * 32 + j] + (tb ? dsum[64 + j] : 0.0f) + exp_fast(m0 - M) * qn[t];
+                    const float inv = 1.0f / (fmaxf(fabsf(den), exp_fast(-(gF[gb + t] + M))) + 1e-6f);
+                    float* orow = a.o + ((int64_t)(t0 + first + c * 64 + t) * a.H + h) * a.Dv + dv0 + w * 32;
+                    if (c * 64 + t < len) {
+#pragma unroll
+                        for (int x = 0; x < 4; ++x) {
+                            const int d = 8 * x + 4 * hl;           // Dv is a multiple of 8: four columns are in or out together
+                            if (dv0 + w * 32 + d < a.Dv)
+                                *(float4*)(orow + d) = make_float4(o[tb][4 * x] * inv, o[tb][4 * x + 1] * inv, o[tb][4 * x + 2] * inv, o[tb][4 * x + 3] * inv);
+                        }
+                    }
+                }
+            }
+        }
         if (MODE == CHUNK_LOCAL) fsum += gF[gb + 63];
         m0 = gF[gb + 63] + Mc;
         if (NB == 1 && c + 1 < nchunks) {

@@ -239,23 +239,29 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowArgs a) {
 }
 
 template <typename T>
-__global__ __launch_bounds__(128) void window_combine_kernel(WindowArgs a) {
+__global__ __launch_bounds__(256) void window_combine_kernel(WindowArgs a) {
+    __shared__ float f[256];                        // a split's share of the result
+    __shared__ float part[4];
     const int64_t bh = blockIdx.x;
     const int64_t b = bh / a.H;
-    const int h = (int)(bh - b * a.H);
-    const float* w = a.ws + bh * a.splits * (a.Dv + 2);
-    float mm = WA_NEG;
-    for (int s = 0; s < a.splits; ++s) mm = fmaxf(mm, w[s * (a.Dv + 2) + a.Dv]);
-    for (int d = threadIdx.x; d < a.Dv; d += 128) {
-        float num = 0.0f, den = 0.0f;
-        for (int s = 0; s < a.splits; ++s) {
-            const float* r = w + s * (a.Dv + 2);
-            const float f = __builtin_amdgcn_exp2f(r[a.Dv] - mm);
-            num += r[d] * f;
-            den += r[a.Dv + 1] * f;
-        }
+    const int h = (int)(bh - b * a.H), tid = threadIdx.x, row = a.Dv + 2;
+    const float* w = a.ws + bh * a.splits * row;
+    const float m = tid < a.splits ? w[tid * row + a.Dv] : WA_NEG, l = tid < a.splits ? w[tid * row + a.Dv + 1] : 0.0f;
+    const float wm = wave_max_f(m);
+    if ((tid & 63) == 0) part[tid >> 6] = wm;
+    __syncthreads();
+    const float mm = fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3]));
+    __syncthreads();
+    const float e = __builtin_amdgcn_exp2f(m - mm);
+    const float inv = 1.0f / block_sum_f(l * e, part, 4);
+    f[tid] = e * inv;
+    __syncthreads();
+    for (int d = tid; d < a.Dv; d += 256) {
+        float num = 0.0f;
+#pragma unroll 8
+        for (int s = 0; s < a.splits; ++s) num += w[s * row + d] * f[s];
         const float gate = sigmoid_f(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
-        st((T*)a.out + bh * a.Dv + d, num / den * gate);
+        st((T*)a.out + bh * a.Dv + d, num * gate);
     }
 }
 
@@ -327,20 +333,40 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
     const int nkept = (max(0, min(a.keep - past, q1 + 1)) + 63) / 64;
     const int wt0 = max(nkept, max(0, q0 - a.size + 1) / 64);
     const int total = nr + nkept + max(0, q1 / 64 + 1 - wt0);
+    // a load instruction of the workgroup covers RL rows; what a lane fetches of them does not depend on the tile, so a tile
+    // whose rows all exist needs scalar addresses only
+    constexpr int RL = 256 / W::PIECES;
+    const int lrow = tid / W::PIECES, lpos = tid % W::PIECES;
+    int kcol[2], vcol[2];                                  // swizzles repeat after 16 rows
+#pragma unroll
+    for (int x = 0; x < 2; ++x) {
+        kcol[x] = min((lpos ^ W::kswz(lrow + x * RL)) * 16, a.Dp * 2 - 16);
+        vcol[x] = min((lpos ^ W::vswz(lrow + x * RL)) * 16, a.Dvp * 2 - 16);
+    }
     auto request = [&](int n, int buf) __attribute__((always_inline)) {
         const bool ring = n < nr;
         const int k0 = 64 * (ring ? n : n - nr < nkept ? n - nr : wt0 + n - nr - nkept);
         const int last = ring ? nring - 1 : len - 1;
         const char* kb = ring ? rk : pk;
         const char* vb = ring ? rv : pv;
-        const int64_t ks = ring ? a.Dp * 2 : (int64_t)a.G * a.Dp * 2, vs = ring ? a.Dvp * 2 : (int64_t)a.G * a.Dvp * 2;
+        const int ks = ring ? a.Dp * 2 : a.G * a.Dp * 2, vs = ring ? a.Dvp * 2 : a.G * a.Dvp * 2;
         const uint32_t dst = lds0 + buf * 2 * W::TILE + w * 1024;
+        if (k0 + 63 <= last) {
+            const char* kt = kb + (int64_t)k0 * ks;
+            const char* vt = vb + (int64_t)k0 * vs;
+            const uint32_t ko = lrow * ks, vo = lrow * vs;
 #pragma unroll
-        for (int x = 0; x < W::LOADS; ++x) {
-            const int p = x * 256 + tid, row = p / W::PIECES, pos = p % W::PIECES;
-            const int64_t key = min(k0 + row, last);
-            load_to_lds16(kb + key * ks + min((pos ^ W::kswz(row)) * 16, a.Dp * 2 - 16), dst + x * 4096);
-            load_to_lds16(vb + key * vs + min((pos ^ W::vswz(row)) * 16, a.Dvp * 2 - 16), dst + W::TILE + x * 4096);
+            for (int x = 0; x < W::LOADS; ++x) {
+                load_to_lds16_at(kt + x * RL * ks, ko + kcol[x & 1], dst + x * 4096);
+                load_to_lds16_at(vt + x * RL * vs, vo + vcol[x & 1], dst + W::TILE + x * 4096);
+            }
+        } else {
+#pragma unroll
+            for (int x = 0; x < W::LOADS; ++x) {
+                const int64_t key = min(k0 + x * RL + lrow, last);
+                load_to_lds16(kb + key * ks + kcol[x & 1], dst + x * 4096);
+                load_to_lds16(vb + key * vs + vcol[x & 1], dst + W::TILE + x * 4096);
+            }
         }
     };
     const int kx = 4 * hl + ((lane & 15) >> 2), jh = (lane >> 4) & 1;   // the transposing read: key of this lane, half of the 32 d
@@ -383,17 +409,13 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
                     const int x = k0 + blk * 32 + 8 * (v >> 2) + 4 * hl + (v & 3);
                     const int pos = ring ? ring_position(x, past, a.keep, a.size) : past + x;
                     const bool see = (ring ? x < nring : pos <= i) && (i - pos < a.size || pos < a.keep);
-                    s[blk][v] = see ? s[blk][v] * a.scale_log2 : WA_NEG;
+                    s[blk][v] = see ? s[blk][v] : WA_NEG;
                 }
-        } else {
-#pragma unroll
-            for (int blk = 0; blk < 2; ++blk)
-#pragma unroll
-                for (int v = 0; v < 16; ++v) s[blk][v] *= a.scale_log2;
         }
         float tm = s[0][0];
 #pragma unroll
         for (int v = 0; v < 16; ++v) tm = fmaxf(tm, fmaxf(s[0][v], s[1][v]));
+        tm = tm > 0.5f * WA_NEG ? tm * a.scale_log2 : WA_NEG;
         // the reference moves only when some row outgrows it by 2^6 (or has none yet)
         if (__builtin_amdgcn_ballot_w64(tm > m + 6.0f) != 0) {
             const float mn = fmaxf(m, fmaxf(tm, __shfl_xor(tm, 32, 64)));
@@ -406,6 +428,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
                 for (int v = 0; v < 16; ++v) o[db][v] *= alpha;
         }
         const float ref = m > 0.5f * WA_NEG ? m : 0.0f;    // a row that has seen nothing: its scores give exp2(-huge) = 0
+        const float sc = a.scale_log2;
 #pragma unroll
         for (int blk = 0; blk < 2; ++blk) {
 #pragma unroll
@@ -413,7 +436,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
                 hy_u32x4 hi, lo;
 #pragma unroll
                 for (int x = 0; x < 4; ++x) {
-                    const float p0 = __builtin_amdgcn_exp2f(s[blk][half * 8 + 2 * x] - ref), p1 = __builtin_amdgcn_exp2f(s[blk][half * 8 + 2 * x + 1] - ref);
+                    const float p0 = __builtin_amdgcn_exp2f(fmaf(s[blk][half * 8 + 2 * x], sc, -ref)), p1 = __builtin_amdgcn_exp2f(fmaf(s[blk][half * 8 + 2 * x + 1], sc, -ref));
                     l += p0 + p1;
                     uint32_t tw[2];
                     split2<2>(p0, p1, tw);
@@ -518,7 +541,7 @@ extern "C" int trimkv_window_decode(const void* q, const void* ring_k, const voi
     a.H = heads; a.G = kv_heads; a.D = dim; a.Dv = vdim; a.Dp = dim_stride; a.Dvp = vdim_stride; a.keep = keep_first; a.size = window;
     a.scale_log2 = scale * 1.4426950408889634f; a.splits = splits; a.ws = workspace;
     if (int rc = window_common(fn, a, batch, dtype)) return rc;
-    if (splits < 1 || splits > 65535 || (splits > 1 && !workspace)) return fail(TRIMKV_ERR_WORKSPACE, "%s: splits=%d needs a workspace", fn, splits);
+    if (splits < 1 || splits > 256 || (splits > 1 && !workspace)) return fail(TRIMKV_ERR_WORKSPACE, "%s: splits=%d needs a workspace", fn, splits);
     const int cap = keep_first + window;
     a.chunk = (cap + splits - 1) / splits;
     const int lanes = ((dim_stride > vdim_stride ? dim_stride : vdim_stride) + 7) / 8;
@@ -531,7 +554,7 @@ extern "C" int trimkv_window_decode(const void* q, const void* ring_k, const voi
         else launch_window_decode<T, 64>(a, batch, s));
     int rc = launch_status(fn);
     if (rc || splits == 1) return rc;
-    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((window_combine_kernel<T>), dim3(batch * heads), dim3(128), 0, s, a));
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((window_combine_kernel<T>), dim3(batch * heads), dim3(256), 0, s, a));
     return launch_status(fn);
 }
 
@@ -550,7 +573,7 @@ extern "C" int trimkv_window_prefill(const void* q, const void* k, const void* v
     hipStream_t s = (hipStream_t)stream;
     const int per = heads / kv_heads, big = dim_stride > vdim_stride ? dim_stride : vdim_stride;
     const bool aligned = !(((uintptr_t)k | (uintptr_t)v) & 15);
-    if (dtype == TRIMKV_BF16 && big <= 256 && per <= 128 && aligned) {
+    if (dtype == TRIMKV_BF16 && big <= 256 && per <= 128 && aligned && scale > 0.0f) {
         a.vec = vdim % 4 == 0 && gate_stride % 4 == 0 && !(((uintptr_t)gate | (uintptr_t)out) & 7);
         const int rc = big <= 64 ? launch_window_prefill<64>(a, batch, max_len, s) : big <= 128 ? launch_window_prefill<128>(a, batch, max_len, s)
                                                                                                : launch_window_prefill<256>(a, batch, max_len, s);

@@ -101,6 +101,25 @@ class MLSTM(nn.Module):
         return self.o(y)
 
 
+class ExpertMatrix:
+    """Where one expert's [n, k] matrix of a checkpoint goes: its blocks in the packed stack (padding stays zero)."""
+
+    def __init__(self, packed: torch.Tensor, n: int, k: int):
+        self.packed, self.shape = packed, (n, k)
+        self.device, self.dtype = packed.device, packed.dtype
+
+    def dim(self) -> int:
+        return 2
+
+    def copy_(self, src: torch.Tensor) -> None:
+        full = torch.zeros(self.packed.shape[0] * 32, self.packed.shape[1] * 16, dtype=self.dtype, device=self.device)
+        full[:self.shape[0], :self.shape[1]] = src
+        self.packed.copy_(ops.pack_matrix(full))
+
+    def value(self) -> torch.Tensor:
+        return ops.unpack_matrix(self.packed)[:self.shape[0], :self.shape[1]]
+
+
 class RoutedExperts(nn.Module):
     """Squared-ReLU experts behind a grouped sigmoid router.  ``forward`` returns the chosen experts' outputs and their
     weights: the weighted sum is taken by whoever adds them to the residual stream."""
@@ -114,13 +133,13 @@ class RoutedExperts(nn.Module):
         wp, fp = ops.padded(width), ops.padded(ff)
         self.router = _param(self.spec.experts, wp, dtype=dtype)
         self.correction = _param(self.spec.experts, dtype=torch.float32)
-        self.up = _param(self.spec.experts, fp, wp, dtype=dtype)
-        self.down = _param(self.spec.experts, wp, fp, dtype=dtype)
+        self.up = _param(self.spec.experts, fp // 32, wp // 16, 2, 32, 8, dtype=dtype)       # packed, see trimkv_moe_gemm
+        self.down = _param(self.spec.experts, wp // 32, fp // 16, 2, 32, 8, dtype=dtype)
 
     def tensors(self) -> Dict[str, torch.Tensor]:
         out = {"router": self.router[:, :self.width], "correction": self.correction}
         for e in range(self.spec.experts):
-            out[f"e{e}.up"], out[f"e{e}.down"] = self.up[e, :self.ff, :self.width], self.down[e, :self.width, :self.ff]
+            out[f"e{e}.up"], out[f"e{e}.down"] = ExpertMatrix(self.up[e], self.ff, self.width), ExpertMatrix(self.down[e], self.width, self.ff)
         return out
 
     def forward(self, x, xh):
@@ -202,7 +221,7 @@ class HybridForCausalLM(GreedyGeneration, nn.Module):
 
     # ---- weights ----------------------------------------------------------------------------------
     def tensors(self) -> Dict[str, torch.Tensor]:
-        """Checkpoint name -> the (part of a) parameter it fills."""
+        """Checkpoint name -> the (part of a) parameter it fills (has ``shape`` and ``copy_``)."""
         out = {"embed": self.model.embed, "final.norm": self.model.norm}
         for i, layer in enumerate(self.model.layers):
             out.update({f"l{i}.{k}": v for k, v in layer.tensors().items()})

@@ -214,13 +214,26 @@ def route(logits: torch.Tensor, correction: torch.Tensor, spec: RouterSpec):
     return ids, weights
 
 
+def pack_matrix(w: torch.Tensor) -> torch.Tensor:
+    """[..., n, k] (multiples of 64) in the blocks trimkv_moe_gemm reads, [..., n / 32, k / 16, 2, 32, 8]."""
+    *lead, n, k = w.shape
+    return w.reshape(*lead, n // 32, 32, k // 16, 2, 8).movedim(-4, -2)
+
+
+def unpack_matrix(p: torch.Tensor) -> torch.Tensor:
+    *lead, nb, kb, _, _, _ = p.shape
+    return p.movedim(-2, -4).reshape(*lead, nb * 32, kb * 16)
+
+
 def experts(x: torch.Tensor, ids: torch.Tensor, up: torch.Tensor, down: torch.Tensor, width: int) -> torch.Tensor:
-    """Rows x [T, k padded], expert ids [T, top] -> [T * top, width]: ``down_e relu(up_e x)^2`` of every (token, choice)."""
+    """Rows x [T, k padded], expert ids [T, top], packed matrices up [E, ff, width] and down [E, width, ff] (``pack_matrix`` of
+    the zero-padded ones) -> [T * top, width]: ``down_e relu(up_e x)^2`` of every (token, choice)."""
     _require(up.dtype, x, up, down)
-    E, ffp, wp = up.shape
+    E, ffp, wp = up.shape[0], up.shape[1] * 32, up.shape[2] * 16
     T, top = ids.shape
     M, dev, lib, st, code = T * top, x.device, _lib.load_hybrid(), _lib.current_stream(x.device), _lib.dtype_code(up.dtype)
-    tile = 128 if up.dtype == torch.bfloat16 and M >= 32 * E else 16      # a few rows per expert: stream the weights past them
+    # rows per expert: many -> tiles of the matrix-bound kernel, a few -> the weights stream past them
+    tile = 16 if up.dtype == torch.float32 else 256 if M >= 96 * E else 32
     most = M if M < E else (M - E) // tile + E
     order = torch.empty(M, dtype=torch.int32, device=dev)
     offsets = torch.empty(E + 1, dtype=torch.int32, device=dev)
