@@ -70,15 +70,15 @@ int trimkv_window_decode(const void* q, const void* ring_k, const void* ring_v, 
 
 /* mLSTM over portions (equations in csrc/mlstm.hip). gates [tokens][2 heads]: W_i h, W_f h without biases.  state
  * [slot][heads][dim][vdim]; norm_state [2][num_slots][heads][dim + 1] (n and m, by parity of the slot's steps).
- * out [tokens][heads][vdim] fp32, before the head norm.  dim up to 512.  workspace: trimkv_mlstm_workspace(...) floats (0: NULL will do), for the states
+ * out [tokens][heads][vdim] in dtype, before the head norm.  dim up to 512.  workspace: trimkv_mlstm_workspace(...) floats (0: NULL will do), for the states
  * between the segments of long bf16 prompts. */
 int64_t trimkv_mlstm_workspace(int batch, int max_len, int heads, int dim, int vdim, int dtype);
 int trimkv_mlstm(const void* proj, int64_t proj_stride, int q_off, int k_off, int v_off, const float* gates, const float* i_bias,
                  const float* f_bias, float gate_cap, float* state, float* norm_state, const int32_t* cu, const int32_t* slots, const int32_t* seen,
-                 float* out, int batch, int max_len, int heads, int dim, int vdim, int num_slots, float q_scale, float* workspace, int dtype, void* stream);
+                 void* out, int batch, int max_len, int heads, int dim, int vdim, int num_slots, float q_scale, float* workspace, int dtype, void* stream);
 
-/* out[t][h][:] = w[h] * o / sqrt(mean(o^2) + eps) * sigmoid(gate), o [tokens][heads][vdim] fp32. */
-int trimkv_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int tokens, int heads, int vdim, float eps, int dtype, void* stream);
+/* out[t][h][:] = w[h] * o / sqrt(mean(o^2) + eps) * sigmoid(gate), o [tokens][heads][vdim] in dtype; norm and gate in fp32. */
+int trimkv_head_norm_gate(const void* o, const void* gate, int64_t gate_stride, const float* w, void* out, int tokens, int heads, int vdim, float eps, int dtype, void* stream);
 
 /* seen[slots[b]] += {cu[b+1] - cu[b], 1}. */
 int trimkv_advance(int32_t* seen, const int32_t* slots, const int32_t* cu, int batch, void* stream);

@@ -28,6 +28,8 @@ __device__ __forceinline__ void st4(bf16_t* p, float4 f) {
 }
 
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
+// for output gates: hardware exponential and reciprocal, a few ulp
+__device__ __forceinline__ float sigmoid_fast(float x) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f)); }
 // log(sigmoid(x)) with the library's exp and log1p
 __device__ __forceinline__ float log_sigmoid_exact(float x) { return fminf(x, 0.0f) - log1pf(expf(-fabsf(x))); }
 

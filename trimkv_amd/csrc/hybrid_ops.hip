@@ -10,6 +10,7 @@
 //   trimkv_head_norm_gate  per-head RMS norm, weight and sigmoid gate behind a recurrence
 //   trimkv_advance         tokens and steps seen per sequence slot
 #include "hybrid.hip.h"
+#include <type_traits>
 
 namespace trimkv {
 
@@ -305,45 +306,52 @@ __global__ __launch_bounds__(256) void ring_store_kernel(const T* k, const T* v,
 
 // ---- behind a recurrence: rms per head, weight, sigmoid gate -------------------------------------
 template <typename T>
-__global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* o, const T* g, int64_t g_stride, const float* w, T* out, int64_t units, int H, int Dv, float eps) {
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const T* o, const T* g, int64_t g_stride, const float* w, T* out, int64_t units, int H, int Dv, float eps) {
     const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (unit >= units) return;
     const int64_t t = unit / H;
     const int h = (int)(unit - t * H), lane = threadIdx.x & 63;
-    const float* src = o + unit * Dv;
+    const T* src = o + unit * Dv;
     const T* gr = g + t * g_stride + h * Dv;
     float ss = 0.0f;
-    for (int i = lane; i < Dv; i += 64) ss += src[i] * src[i];
+    for (int i = lane; i < Dv; i += 64) { const float f = ld(src + i); ss += f * f; }
     const float inv = 1.0f / sqrtf(wave_sum_f(ss) / (float)Dv + eps);
-    for (int i = lane; i < Dv; i += 64) st(out + unit * Dv + i, src[i] * inv * w[h * Dv + i] * sigmoid_f(ld(gr + i)));
+    for (int i = lane; i < Dv; i += 64) st(out + unit * Dv + i, ld(src + i) * inv * w[h * Dv + i] * sigmoid_fast(ld(gr + i)));
 }
 
-// Dv a multiple of 4 up to 256 NV: the row is held in registers
-template <typename T, int NV>
-__global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(const float* o, const T* g, int64_t g_stride, const float* w, T* out, int64_t units, int H, int Dv, float eps) {
-    const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (unit >= units) return;
-    const int64_t t = unit / H;
-    const int h = (int)(unit - t * H), lane = threadIdx.x & 63;
-    float4 s[NV], gt[NV], wt[NV];
-    float ss = 0.0f;
+// Dv a multiple of 8: LH lanes with eight values each per head, 64 / LH heads per wavefront and pass, two passes on their way
+// together
+template <typename T, int LH>
+__global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(const T* o, const T* g, int64_t g_stride, const float* w, T* out, int64_t units, int H, int Dv, float eps) {
+    constexpr int PER = 4 * 64 / LH, U = 2;
+    const int sub = threadIdx.x / LH, i = (threadIdx.x % LH) * 8;
+    const bool in = i < Dv;
+    Eight s[U], gt[U];
+    int64_t unit[U];
+    int h[U];
 #pragma unroll
-    for (int v = 0; v < NV; ++v) {
-        const int i = (v * 64 + lane) * 4;
-        s[v] = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (i < Dv) {
-            s[v] = ld4(o + unit * Dv + i);
-            gt[v] = ld4(g + t * g_stride + h * Dv + i);
-            wt[v] = ld4(w + h * Dv + i);
-        }
-        ss += s[v].x * s[v].x + s[v].y * s[v].y + s[v].z * s[v].z + s[v].w * s[v].w;
+    for (int u = 0; u < U; ++u) {
+        unit[u] = min((int64_t)blockIdx.x * PER * U + u * PER + sub, units - 1);      // past the end: the last one again, same values
+        const int64_t t = unit[u] / H;
+        h[u] = (int)(unit[u] - t * H);
+        s[u] = ld8(o + unit[u] * Dv + (in ? i : 0));
+        gt[u] = ld8(g + t * g_stride + h[u] * Dv + (in ? i : 0));
     }
-    const float inv = 1.0f / sqrtf(wave_sum_f(ss) / (float)Dv + eps);
 #pragma unroll
-    for (int v = 0; v < NV; ++v) {
-        const int i = (v * 64 + lane) * 4;
-        if (i < Dv) st4(out + unit * Dv + i, make_float4(s[v].x * inv * wt[v].x * sigmoid_f(gt[v].x), s[v].y * inv * wt[v].y * sigmoid_f(gt[v].y),
-                                                         s[v].z * inv * wt[v].z * sigmoid_f(gt[v].z), s[v].w * inv * wt[v].w * sigmoid_f(gt[v].w)));
+    for (int u = 0; u < U; ++u) {
+        float ss = 0.0f;
+#pragma unroll
+        for (int x = 0; x < 8; ++x) ss += s[u].f[x] * s[u].f[x];
+        if (!in) ss = 0.0f;
+#pragma unroll
+        for (int d = LH / 2; d > 0; d >>= 1) ss += __shfl_xor(ss, d, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)Dv + eps);
+        if (in) {
+            const Eight wt = ld8(w + h[u] * Dv + i);
+#pragma unroll
+            for (int x = 0; x < 8; ++x) s[u].f[x] *= inv * wt.f[x] * sigmoid_fast(gt[u].f[x]);
+            st8(out + unit[u] * Dv + i, s[u]);
+        }
     }
 }
 
@@ -454,20 +462,25 @@ extern "C" int trimkv_ring_store(const void* k, const void* v, const int32_t* cu
     return launch_status(fn);
 }
 
-extern "C" int trimkv_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int tokens, int heads, int vdim, float eps, int dtype, void* stream) {
+extern "C" int trimkv_head_norm_gate(const void* o, const void* gate, int64_t gate_stride, const float* w, void* out, int tokens, int heads, int vdim, float eps, int dtype, void* stream) {
     const char* fn = "trimkv_head_norm_gate";
     if (!o || !gate || !w || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
     HY_CHECK_DTYPE(fn, dtype);
     if (tokens <= 0 || heads <= 0 || vdim <= 0) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d heads=%d vdim=%d", fn, tokens, heads, vdim);
     const int64_t units = (int64_t)tokens * heads;
-    if (vdim % 4 == 0 && vdim <= 512 && gate_stride % 4 == 0 && !(((uintptr_t)o | (uintptr_t)gate | (uintptr_t)w | (uintptr_t)out) & 15)) {
-        const dim3 grid((unsigned)((units + 3) / 4));
-        HY_BY_DTYPE(dtype, T,
-            if (vdim <= 256) hipLaunchKernelGGL((head_norm_gate_vec_kernel<T, 1>), grid, dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps);
-            else hipLaunchKernelGGL((head_norm_gate_vec_kernel<T, 2>), grid, dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
+    if (vdim % 8 == 0 && vdim <= 512 && gate_stride % 8 == 0 && !(((uintptr_t)o | (uintptr_t)gate | (uintptr_t)w | (uintptr_t)out) & 15)) {
+        auto go = [&](auto lh) {
+            constexpr int LH = decltype(lh)::value, PER = 4 * 64 / LH * 2;
+            HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((head_norm_gate_vec_kernel<T, LH>), dim3((unsigned)((units + PER - 1) / PER)), dim3(256), 0, (hipStream_t)stream,
+                                                     (const T*)o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
+        };
+        if (vdim <= 64) go(std::integral_constant<int, 8>{});
+        else if (vdim <= 128) go(std::integral_constant<int, 16>{});
+        else if (vdim <= 256) go(std::integral_constant<int, 32>{});
+        else go(std::integral_constant<int, 64>{});
         return launch_status(fn);
     }
-    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((head_norm_gate_kernel<T>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((head_norm_gate_kernel<T>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, (hipStream_t)stream, (const T*)o, (const T*)gate, gate_stride, w, (T*)out, units, heads, vdim, eps));
     return launch_status(fn);
 }
 

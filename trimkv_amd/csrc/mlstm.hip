@@ -21,7 +21,7 @@ struct MlstmArgs {
     const float* ib; const float* fb; float cap;
     float* S; float* nm;                                        // nm: [2][slots][H][D + 1]
     const int32_t* cu; const int32_t* slots; const int32_t* seen;
-    float* o;                                                   // [T][H][Dv]
+    void* o;                                                    // [T][H][Dv] in the activations' type
     int H, D, Dv, nslots;
     float qscale;
 };
@@ -81,7 +81,7 @@ __global__ __launch_bounds__(256) void mlstm_recurrent_kernel(MlstmArgs a) {
         __syncthreads();
         if (w == 0 && cin) {
             num = red[lane] + red[64 + lane] + red[128 + lane] + red[192 + lane];
-            a.o[(tok * a.H + h) * a.Dv + col] = num / (fmaxf(fabsf(qn), expf(-m)) + 1e-6f);
+            st((T*)a.o + (tok * a.H + h) * a.Dv + col, num / (fmaxf(fabsf(qn), expf(-m)) + 1e-6f));
         }
         __syncthreads();                          // red, part, q and k are free again
     }
@@ -102,8 +102,9 @@ __global__ __launch_bounds__(256) void mlstm_recurrent_kernel(MlstmArgs a) {
 //   m_t = F_t + M_t,   o_t ~ sum_{s<=t} exp(d_s - M_t) (q_t.k_s) v_s + exp(m_0 - M_t) S_0^T q_t,   n.q alike without v,
 //   S_C = exp(m_0 - M_C) S_0 + sum_s exp(d_s - M_C) k_s v_s^T.
 //
-// q, k, v are bf16; everything that multiplies them (S, the weighted scores, the weighted v) is fp32 and enters the matrix
-// cores as three bf16 terms, so products and sums are fp32.  A workgroup owns 128 value columns of one head, a wavefront 32:
+// q, k, v are bf16; everything that multiplies them is fp32 and enters the matrix cores as a sum of bf16 terms: the weighted v
+// that goes into the state as three (fp32 products), S and the weighted scores on their way to an output as two (17 bits).
+// The state itself stays in fp32 accumulators.  A workgroup owns 128 value columns of one head, a wavefront 32:
 // its part of S stays in the accumulators, whose layout (column = lane % 32, rows 8 (v / 4) + 4 half + v % 4) is the operand
 // layout of S_0^T q with k taken in the order 4 half + 0..3, 8 + 4 half + 0..3 of every 16.  The same order is used along s
 // (V and K are read transposed, ds_read_b64_tr_b16).
@@ -119,11 +120,11 @@ enum { CHUNK_WHOLE = 0, CHUNK_LOCAL = 1, CHUNK_OUTPUT = 2 };
 
 template <int DKT>
 struct ChunkCfg {
-    static constexpr int DK = 32 * DKT, NBUF = DKT <= 4 ? 2 : 1;
+    static constexpr int DK = 32 * DKT, NBUF = 1;       // two workgroups fit a CU and hide each other's loads
     static constexpr int QB = 64 * DK * 2, VB = 64 * 256, BUF = 2 * QB + VB;
     static constexpr int PROW = 144, PPLANE = 64 * PROW;
-    static constexpr int P0 = NBUF * BUF, F0 = P0 + 3 * PPLANE;
-    static constexpr int LDS = F0 + (6 * 64 + DK + 64 + 96) * 4;
+    static constexpr int P0 = NBUF * BUF, F0 = P0 + 2 * PPLANE;
+    static constexpr int LDS = F0 + (6 * 64 + DK + 64 + 96 + 256) * 4;
     // position of 16-byte piece c of row r: rows that one read instruction touches together fall on different banks
     static __device__ __forceinline__ int swz(int r) {
         return DK == 32 ? (r >> 2) & 3 : DK == 64 ? (((r >> 1) & 1) << 2) | ((r >> 2) & 3) : ((r & 3) << 2) | ((r >> 2) & 3);
@@ -141,10 +142,13 @@ __device__ __forceinline__ float wave_scan_max(float v, int lane) {
     for (int d = 1; d < 64; d <<= 1) { const float o = __shfl_up(v, d, 64); if (lane >= d) v = fmaxf(v, o); }
     return v;
 }
-__device__ __forceinline__ float exp_fast(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+// The chunk kernels keep gates and stabilisers in units of log 2, so that an exponential is one instruction; the state's m is
+// converted on the way in and out.
+constexpr float LOG2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
+__device__ __forceinline__ float exp_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
-template <int DKT, int MODE>
-__global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
+template <int DKT, int MODE, bool FULL>     // FULL: dim is exactly 32 DKT
+__global__ __launch_bounds__(256, DKT <= 4 ? 2 : 1) void mlstm_chunk_kernel(ChunkArgs ca) {
     using C = ChunkCfg<DKT>;
     constexpr int DK = C::DK, NB = C::NBUF;
     const MlstmArgs& a = ca.a;
@@ -154,6 +158,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
     float* const gF = (float*)(ck_lds + C::F0);      // [2][64] each
     float* const gD = gF + 128; float* const gM = gD + 128;
     float* const n = gM + 128; float* const qn = n + DK; float* const dsum = qn + 64;
+    float* const wgt = dsum + 96;                     // [4][64]: every wavefront's own copy of exp(d_s - M_C)
     const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane & 31, hl = lane >> 5;
     const int vt = (a.Dv + 127) / 128, seg = blockIdx.x / vt, dv0 = (blockIdx.x % vt) * 128, h = blockIdx.y, b = blockIdx.z;
     const int t0 = a.cu[b], len_all = a.cu[b + 1] - t0;
@@ -179,10 +184,10 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
 #pragma unroll
             for (int v = 0; v < 16; ++v) {
                 const int d = db * 32 + 8 * (v >> 2) + 4 * hl + (v & 3);
-                S[db][v] = zero || d >= a.D || col >= a.Dv ? 0.0f : src[(int64_t)d * a.Dv + col];
+                S[db][v] = zero || (!FULL && d >= a.D) || col >= a.Dv ? 0.0f : src[(int64_t)d * a.Dv + col];
             }
         for (int d = tid; d < DK; d += 256) n[d] = zero || d >= a.D ? 0.0f : nsrc[d];
-        m0 = MODE == CHUNK_LOCAL ? -1.0e30f : MODE == CHUNK_OUTPUT ? ca.seg_m[sat] : fresh ? 0.0f : a.nm[parity * copy + at + a.D];
+        m0 = MODE == CHUNK_LOCAL ? -1.0e30f : MODE == CHUNK_OUTPUT ? ca.seg_m[sat] : fresh ? 0.0f : a.nm[parity * copy + at + a.D] * LOG2E;
     }
     const bf16_t* base = (const bf16_t*)a.p + (int64_t)(t0 + first) * a.p_stride;
     auto request = [&](int c, int buf) __attribute__((always_inline)) {
@@ -210,8 +215,8 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
     };
     auto gates = [&](int c, int buf) __attribute__((always_inline)) {
         const int t = c * 64 + lane;
-        const float li = t < len ? log_input_gate(zi + ib, a.cap) : -1.0e30f;
-        const float lf = t < len ? log_forget_gate(zf + fb, a.cap) : 0.0f;
+        const float li = t < len ? log_input_gate(zi + ib, a.cap) * LOG2E : -1.0e30f;
+        const float lf = t < len ? log_forget_gate(zf + fb, a.cap) * LOG2E : 0.0f;
         const float F = wave_scan_add(lf, lane), d = li - F;
         gF[buf * 64 + lane] = F;
         gD[buf * 64 + lane] = d;
@@ -238,6 +243,8 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
         if (NB == 2 && c + 1 < nchunks) request(c + 1, buf ^ 1);
         if (w == 3 && c + 1 < nchunks) { gates(c + 1, (c + 1) & 1); fetch_gates(c + 2); }
         const float Mc = fmaxf(m0, gM[gb + 63]);
+        float* const ws = wgt + w * 64;
+        ws[lane] = exp_fast(gD[gb + lane] - Mc);
         hy_f32x16 o[2];
         if (MODE != CHUNK_LOCAL) {
             if (w < 3) {                              // scores, weighted: blocks (s, t) = (0, 0), (0, 1), (1, 1)
@@ -250,7 +257,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                     const int kr = sb * 32 + j, qr = tb * 32 + j, pcs = 2 * ks + hl;
                     const hy_bf16x8 kf = *(const HY_LDS hy_bf16x8*)(lds3 + off + C::QB + kr * DK * 2 + ((pcs ^ C::swz(kr)) << 4));
                     hy_u32x4 qf = *(const HY_LDS hy_u32x4*)(lds3 + off + qr * DK * 2 + ((pcs ^ C::swz(qr)) << 4));
-                    if (pcs * 8 >= a.D) qf = hy_u32x4{0u, 0u, 0u, 0u};
+                    if (!FULL && pcs * 8 >= a.D) qf = hy_u32x4{0u, 0u, 0u, 0u};
                     p = mfma32(kf, __builtin_bit_cast(hy_bf16x8, qf), p);
                 }
                 const int t = tb * 32 + j;
@@ -267,11 +274,11 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                         q[y] = s <= t ? p[4 * x + y] * a.qscale * exp_fast(dd[y] - M) : 0.0f;
                         sum += q[y];
                     }
-                    uint32_t e0[3], e1[3];
-                    split2<3>(q[0], q[1], e0);
-                    split2<3>(q[2], q[3], e1);
+                    uint32_t e0[2], e1[2];
+                    split2<2>(q[0], q[1], e0);
+                    split2<2>(q[2], q[3], e1);
 #pragma unroll
-                    for (int e = 0; e < 3; ++e)
+                    for (int e = 0; e < 2; ++e)
                         *(uint2*)(ck_lds + C::P0 + e * C::PPLANE + t * C::PROW + (sb * 32 + 8 * x + 4 * hl) * 2) = make_uint2(e0[e], e1[e]);
                 }
                 sum += __shfl_xor(sum, 32, 64);
@@ -293,22 +300,22 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                 for (int db = 0; db < DKT; ++db)
 #pragma unroll
                     for (int st_ = 0; st_ < 2; ++st_) {
-                        uint32_t e0[3], e1[3], e2[3], e3[3];
-                        split2<3>(S[db][8 * st_], S[db][8 * st_ + 1], e0);
-                        split2<3>(S[db][8 * st_ + 2], S[db][8 * st_ + 3], e1);
-                        split2<3>(S[db][8 * st_ + 4], S[db][8 * st_ + 5], e2);
-                        split2<3>(S[db][8 * st_ + 6], S[db][8 * st_ + 7], e3);
+                        uint32_t e0[2], e1[2], e2[2], e3[2];
+                        split2<2>(S[db][8 * st_], S[db][8 * st_ + 1], e0);
+                        split2<2>(S[db][8 * st_ + 2], S[db][8 * st_ + 3], e1);
+                        split2<2>(S[db][8 * st_ + 4], S[db][8 * st_ + 5], e2);
+                        split2<2>(S[db][8 * st_ + 6], S[db][8 * st_ + 7], e3);
                         const int pcs = db * 4 + st_ * 2;
 #pragma unroll
                         for (int tb = 0; tb < 2; ++tb) {
                             const int r = tb * 32 + j;
                             const HY_LDS char* qp = lds3 + off + r * DK * 2 + hl * 8;
                             hy_u32x2 lo = *(const HY_LDS hy_u32x2*)(qp + ((pcs ^ C::swz(r)) << 4)), hi = *(const HY_LDS hy_u32x2*)(qp + (((pcs + 1) ^ C::swz(r)) << 4));
-                            if (pcs * 8 >= a.D) lo = hy_u32x2{0u, 0u};
-                            if (pcs * 8 + 8 >= a.D) hi = hy_u32x2{0u, 0u};
+                            if (!FULL && pcs * 8 >= a.D) lo = hy_u32x2{0u, 0u};
+                            if (!FULL && pcs * 8 + 8 >= a.D) hi = hy_u32x2{0u, 0u};
                             const hy_bf16x8 qf = __builtin_bit_cast(hy_bf16x8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3));
 #pragma unroll
-                            for (int e = 2; e >= 0; --e)
+                            for (int e = 1; e >= 0; --e)
                                 o[tb] = mfma32(__builtin_bit_cast(hy_bf16x8, (hy_u32x4){e0[e], e1[e], e2[e], e3[e]}), qf, o[tb]);
                         }
                     }
@@ -335,7 +342,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                     for (int tb = 0; tb < 2; ++tb) {
                         if (tb == 0 && st_ >= 2) continue;
 #pragma unroll
-                        for (int e = 2; e >= 0; --e) {
+                        for (int e = 1; e >= 0; --e) {
                             const char* pp = ck_lds + C::P0 + e * C::PPLANE + (tb * 32 + j) * C::PROW + (16 * st_ + 4 * hl) * 2;
                             const uint2 lo = *(const uint2*)pp, hi = *(const uint2*)(pp + 16);
                             o[tb] = mfma32(vf, __builtin_bit_cast(hy_bf16x8, (hy_u32x4){lo.x, lo.y, hi.x, hi.y}), o[tb]);
@@ -343,12 +350,12 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                     }
                 }
                 const hy_u32x4 vr = __builtin_bit_cast(hy_u32x4, vf);
-                const float4 d0 = *(const float4*)(gD + gb + 16 * st_ + 4 * hl), d1 = *(const float4*)(gD + gb + 16 * st_ + 4 * hl + 8);
+                const float4 d0 = *(const float4*)(ws + 16 * st_ + 4 * hl), d1 = *(const float4*)(ws + 16 * st_ + 4 * hl + 8);
                 uint32_t e0[3], e1[3], e2[3], e3[3];
-                split2<3>(__uint_as_float(vr[0] << 16) * exp_fast(d0.x - Mc), __uint_as_float(vr[0] & 0xffff0000u) * exp_fast(d0.y - Mc), e0);
-                split2<3>(__uint_as_float(vr[1] << 16) * exp_fast(d0.z - Mc), __uint_as_float(vr[1] & 0xffff0000u) * exp_fast(d0.w - Mc), e1);
-                split2<3>(__uint_as_float(vr[2] << 16) * exp_fast(d1.x - Mc), __uint_as_float(vr[2] & 0xffff0000u) * exp_fast(d1.y - Mc), e2);
-                split2<3>(__uint_as_float(vr[3] << 16) * exp_fast(d1.z - Mc), __uint_as_float(vr[3] & 0xffff0000u) * exp_fast(d1.w - Mc), e3);
+                split2<3>(__uint_as_float(vr[0] << 16) * d0.x, __uint_as_float(vr[0] & 0xffff0000u) * d0.y, e0);
+                split2<3>(__uint_as_float(vr[1] << 16) * d0.z, __uint_as_float(vr[1] & 0xffff0000u) * d0.w, e1);
+                split2<3>(__uint_as_float(vr[2] << 16) * d1.x, __uint_as_float(vr[2] & 0xffff0000u) * d1.y, e2);
+                split2<3>(__uint_as_float(vr[3] << 16) * d1.z, __uint_as_float(vr[3] & 0xffff0000u) * d1.w, e3);
 #pragma unroll
                 for (int db = 0; db < DKT; ++db) {
                     const hy_bf16x8 kf = tr_read(off + C::QB, DK * 2, ksw0, ksw1, st_, db);
@@ -371,9 +378,9 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                     for (int i = 0; i < 16; ++i) {
                         const int s = qt * 16 + i;
                         const uint32_t k2 = *(const HY_LDS uint32_t*)(lds3 + off + C::QB + s * DK * 2 + (((d >> 3) ^ C::swz(s)) << 4) + (d & 7) * 2);
-                        const float ws = exp_fast(gD[gb + s] - Mc);
-                        x += ws * __uint_as_float(k2 << 16);
-                        y += ws * __uint_as_float(k2 & 0xffff0000u);
+                        const float f = ws[s];
+                        x += f * __uint_as_float(k2 << 16);
+                        y += f * __uint_as_float(k2 & 0xffff0000u);
                     }
                     x += __shfl_xor(x, 16, 64); y += __shfl_xor(y, 16, 64);
                     x += __shfl_xor(x, 32, 64); y += __shfl_xor(y, 32, 64);
@@ -390,13 +397,13 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
                     const float M = fmaxf(m0, gM[gb + t]);
                     const float den = dsum[tb * 32 + j] + (tb ? dsum[64 + j] : 0.0f) + exp_fast(m0 - M) * qn[t];
                     const float inv = 1.0f / (fmaxf(fabsf(den), exp_fast(-(gF[gb + t] + M))) + 1e-6f);
-                    float* orow = a.o + ((int64_t)(t0 + first + c * 64 + t) * a.H + h) * a.Dv + dv0 + w * 32;
+                    bf16_t* orow = (bf16_t*)a.o + ((int64_t)(t0 + first + c * 64 + t) * a.H + h) * a.Dv + dv0 + w * 32;
                     if (c * 64 + t < len) {
 #pragma unroll
                         for (int x = 0; x < 4; ++x) {
                             const int d = 8 * x + 4 * hl;           // Dv is a multiple of 8: four columns are in or out together
                             if (dv0 + w * 32 + d < a.Dv)
-                                *(float4*)(orow + d) = make_float4(o[tb][4 * x] * inv, o[tb][4 * x + 1] * inv, o[tb][4 * x + 2] * inv, o[tb][4 * x + 3] * inv);
+                                *(uint2*)(orow + d) = make_uint2(pack2(o[tb][4 * x] * inv, o[tb][4 * x + 1] * inv), pack2(o[tb][4 * x + 2] * inv, o[tb][4 * x + 3] * inv));
                         }
                     }
                 }
@@ -418,7 +425,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
 #pragma unroll
             for (int v = 0; v < 16; ++v) {
                 const int d = db * 32 + 8 * (v >> 2) + 4 * hl + (v & 3);
-                if (d < a.D) dst[(int64_t)d * a.Dv + col] = S[db][v];
+                if (FULL || d < a.D) dst[(int64_t)d * a.Dv + col] = S[db][v];
             }
     }
     if (dv0 == 0) {
@@ -426,7 +433,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(ChunkArgs ca) {
         for (int d = tid; d < a.D; d += 256) nd[d] = n[d];
         if (tid == 0) {
             if (MODE == CHUNK_LOCAL) { ca.seg_g[2 * sat] = fsum; ca.seg_g[2 * sat + 1] = m0; }
-            else nd[a.D] = m0;
+            else nd[a.D] = m0 * LN2;
         }
     }
 }
@@ -443,7 +450,7 @@ __global__ __launch_bounds__(256) void mlstm_join_kernel(ChunkArgs ca) {
     const int64_t copy = (int64_t)a.nslots * a.H * (a.D + 1), at = ((int64_t)slot * a.H + h) * (a.D + 1);
     const float* in = a.nm + parity * copy + at;
     float* S = a.S + ((int64_t)slot * a.H + h) * nS;
-    float m = fresh ? 0.0f : in[a.D], cur = fresh ? 0.0f : e < nS ? S[e] : in[e - nS];
+    float m = fresh ? 0.0f : in[a.D] * LOG2E, cur = fresh ? 0.0f : e < nS ? S[e] : in[e - nS];
     const int64_t s0 = ((int64_t)b * a.H + h) * ca.nseg;
     for (int s = 0; s < ca.nseg && s * ca.seg_len < len; ++s) {
         float* p = e < nS ? ca.seg_S + (s0 + s) * nS + e : ca.seg_n + (s0 + s) * a.D + (e - nS);
@@ -456,30 +463,30 @@ __global__ __launch_bounds__(256) void mlstm_join_kernel(ChunkArgs ca) {
     }
     float* out = a.nm + (1 - parity) * copy + at;
     if (e < nS) S[e] = cur; else out[e - nS] = cur;
-    if (e == 0) out[a.D] = m;
+    if (e == 0) out[a.D] = m * LN2;
 }
 
-template <int DKT, int MODE>
+template <int DKT, int MODE, bool FULL>
 static int launch_chunk(const ChunkArgs& c, dim3 grid, hipStream_t s) {
     static bool opted_in[64] = {};
     int dev = 0;
     if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) dev = -1;
     if (dev < 0 || !opted_in[dev]) {
-        hipError_t e = hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DKT, MODE>, hipFuncAttributeMaxDynamicSharedMemorySize, ChunkCfg<DKT>::LDS);
+        hipError_t e = hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DKT, MODE, FULL>, hipFuncAttributeMaxDynamicSharedMemorySize, ChunkCfg<DKT>::LDS);
         if (e != hipSuccess) return (int)e;
         if (dev >= 0) opted_in[dev] = true;
     }
-    hipLaunchKernelGGL((mlstm_chunk_kernel<DKT, MODE>), grid, dim3(256), ChunkCfg<DKT>::LDS, s, c);
+    hipLaunchKernelGGL((mlstm_chunk_kernel<DKT, MODE, FULL>), grid, dim3(256), ChunkCfg<DKT>::LDS, s, c);
     return 0;
 }
-template <int DKT>
+template <int DKT, bool FULL>
 static int launch_chunked(const ChunkArgs& c, int batch, hipStream_t s) {
     const MlstmArgs& a = c.a;
     const int vt = (a.Dv + 127) / 128;
-    if (c.nseg == 1) return launch_chunk<DKT, CHUNK_WHOLE>(c, dim3(vt, a.H, batch), s);
-    if (int rc = launch_chunk<DKT, CHUNK_LOCAL>(c, dim3(vt * c.nseg, a.H, batch), s)) return rc;
+    if (c.nseg == 1) return launch_chunk<DKT, CHUNK_WHOLE, FULL>(c, dim3(vt, a.H, batch), s);
+    if (int rc = launch_chunk<DKT, CHUNK_LOCAL, FULL>(c, dim3(vt * c.nseg, a.H, batch), s)) return rc;
     hipLaunchKernelGGL(mlstm_join_kernel, dim3((a.D * a.Dv + a.D + 255) / 256, a.H, batch), dim3(256), 0, s, c);
-    return launch_chunk<DKT, CHUNK_OUTPUT>(c, dim3(vt * c.nseg, a.H, batch), s);
+    return launch_chunk<DKT, CHUNK_OUTPUT, FULL>(c, dim3(vt * c.nseg, a.H, batch), s);
 }
 // the chunk kernel reads 16-byte pieces of rows and holds one head's query/key features in registers
 static bool chunk_fits(int64_t proj_stride, int q_off, int k_off, int v_off, int dim, int vdim, int dtype, int max_len, const void* proj) {
@@ -505,7 +512,7 @@ extern "C" int64_t trimkv_mlstm_workspace(int batch, int max_len, int heads, int
 
 extern "C" int trimkv_mlstm(const void* proj, int64_t proj_stride, int q_off, int k_off, int v_off, const float* gates, const float* i_bias,
                             const float* f_bias, float gate_cap, float* state, float* norm_state, const int32_t* cu, const int32_t* slots, const int32_t* seen,
-                            float* out, int batch, int max_len, int heads, int dim, int vdim, int num_slots, float q_scale, float* workspace, int dtype, void* stream) {
+                            void* out, int batch, int max_len, int heads, int dim, int vdim, int num_slots, float q_scale, float* workspace, int dtype, void* stream) {
     const char* fn = "trimkv_mlstm";
     if (!proj || !gates || !i_bias || !f_bias || !state || !norm_state || !cu || !slots || !seen || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
     HY_CHECK_DTYPE(fn, dtype);
@@ -524,8 +531,12 @@ extern "C" int trimkv_mlstm(const void* proj, int64_t proj_stride, int q_off, in
             const int64_t n = (int64_t)batch * heads * c.nseg;
             c.seg_S = workspace; c.seg_n = c.seg_S + n * dim * vdim; c.seg_g = c.seg_n + n * dim; c.seg_m = c.seg_g + 2 * n;
         }
-        const int rc = dim <= 32 ? launch_chunked<1>(c, batch, s) : dim <= 64 ? launch_chunked<2>(c, batch, s) : dim <= 128 ? launch_chunked<4>(c, batch, s)
-                                                                                                               : launch_chunked<8>(c, batch, s);
+        int rc;
+        if (dim == 256) rc = launch_chunked<8, true>(c, batch, s);
+        else if (dim == 128) rc = launch_chunked<4, true>(c, batch, s);
+        else if (dim == 64) rc = launch_chunked<2, true>(c, batch, s);
+        else rc = dim <= 32 ? launch_chunked<1, false>(c, batch, s) : dim < 64 ? launch_chunked<2, false>(c, batch, s) : dim < 128 ? launch_chunked<4, false>(c, batch, s)
+                                                                                                                     : launch_chunked<8, false>(c, batch, s);
         if (rc) return fail(rc, "%s: hipFuncSetAttribute failed (%d)", fn, rc);
         return launch_status(fn);
     }

@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WindowArgs a) {
 #pragma unroll
     for (int c = 0; c < 8; ++c) {
         const int d = c * 64 + lane;
-        if (d < a.Dv) st(o + d, acc[c] * inv * sigmoid_f(ld(gr + d)));
+        if (d < a.Dv) st(o + d, acc[c] * inv * sigmoid_fast(ld(gr + d)));
     }
 }
 
@@ -228,7 +228,7 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowArgs a) {
         }
         const int h = g * per + h0 + x;
         if (a.splits == 1) {
-            const float gate = sigmoid_f(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
+            const float gate = sigmoid_fast(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
             st((T*)a.out + ((int64_t)b * a.H + h) * a.Dv + d, num / den * gate);
         } else {
             float* w = a.ws + (((int64_t)b * a.H + h) * a.splits + split) * (a.Dv + 2);
@@ -260,7 +260,7 @@ __global__ __launch_bounds__(256) void window_combine_kernel(WindowArgs a) {
         float num = 0.0f;
 #pragma unroll 8
         for (int s = 0; s < a.splits; ++s) num += w[s * row + d] * f[s];
-        const float gate = sigmoid_f(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
+        const float gate = sigmoid_fast(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
         st((T*)a.out + bh * a.Dv + d, num * gate);
     }
 }
@@ -281,7 +281,7 @@ struct WindowTile {
 };
 
 template <int D>
-__global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
+__global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(WindowArgs a) {
     using W = WindowTile<D>;
     constexpr int KS = D / 16, DB = D / 32;
     extern __shared__ __attribute__((aligned(16))) char wa_lds[];
@@ -391,26 +391,56 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
         if (!ring && k0 > tw1) continue;                   // wavefront-uniform: nothing of the tile is visible yet
         if (!ring && k0 + 63 <= tw0 - a.size && past + k0 >= a.keep) continue;   // ... or any more
         const int off = (n & 1) * 2 * W::TILE;
+        // operands are requested AHEAD steps before the MFMA that takes them; the fences keep the compiler from moving them back
+        constexpr int AHEAD = 3;
         hy_f32x16 s[2];
 #pragma unroll
-        for (int blk = 0; blk < 2; ++blk) {
+        for (int v = 0; v < 16; ++v) s[0][v] = s[1][v] = 0.0f;
+        {
+            hy_bf16x8 kf[2 * KS];
 #pragma unroll
-            for (int v = 0; v < 16; ++v) s[blk][v] = 0.0f;
+            for (int x = 0; x < AHEAD; ++x) kf[x] = k_frag(off, x & 1, x >> 1);
 #pragma unroll
-            for (int ks = 0; ks < KS; ++ks) s[blk] = mfma32(k_frag(off, blk, ks), qf[ks], s[blk]);
+            for (int x = 0; x < 2 * KS; ++x) {
+                if (x + AHEAD < 2 * KS) kf[x + AHEAD] = k_frag(off, (x + AHEAD) & 1, (x + AHEAD) >> 1);
+                s[x & 1] = mfma32(kf[x], qf[x >> 1], s[x & 1]);
+                __builtin_amdgcn_sched_barrier(0);
+            }
         }
+        hy_bf16x8 vf[4 * DB];
+#pragma unroll
+        for (int x = 0; x < AHEAD; ++x) vf[x] = v_frag(off, x / DB, x % DB);
         const bool whole = !ring && k0 + 63 <= tw0 && (k0 > tw1 - a.size || past + k0 + 63 < a.keep);
         if (!whole) {
             asm volatile("" :::);                          // keeps this a branch
-#pragma unroll
-            for (int blk = 0; blk < 2; ++blk)
-#pragma unroll
+            if (ring) {
+#pragma unroll 1
                 for (int v = 0; v < 16; ++v) {
-                    const int x = k0 + blk * 32 + 8 * (v >> 2) + 4 * hl + (v & 3);
-                    const int pos = ring ? ring_position(x, past, a.keep, a.size) : past + x;
-                    const bool see = (ring ? x < nring : pos <= i) && (i - pos < a.size || pos < a.keep);
-                    s[blk][v] = see ? s[blk][v] : WA_NEG;
+                    // (rarely taken: a loop over registers through a compare, not 32 copies of the slot arithmetic)
+                    const int x = k0 + 8 * (v >> 2) + 4 * hl + (v & 3);
+                    bool see[2];
+#pragma unroll
+                    for (int blk = 0; blk < 2; ++blk) {
+                        const int slot_ = x + 32 * blk, pos = ring_position(slot_, past, a.keep, a.size);
+                        see[blk] = slot_ < nring && (i - pos < a.size || pos < a.keep);
+                    }
+#pragma unroll
+                    for (int u = 0; u < 16; ++u) {
+                        s[0][u] = u == v && !see[0] ? WA_NEG : s[0][u];
+                        s[1][u] = u == v && !see[1] ? WA_NEG : s[1][u];
+                    }
                 }
+            } else {
+                const int x1 = i - past, x0 = x1 - a.size, xk = a.keep - past;    // rows up to x1 and beyond x0 or below xk
+#pragma unroll
+                for (int blk = 0; blk < 2; ++blk)
+#pragma unroll
+                    for (int v = 0; v < 16; ++v) {
+                        const int x = k0 + blk * 32 + 8 * (v >> 2) + 4 * hl + (v & 3);
+                        const bool see = (x <= x1) & ((x > x0) | (x < xk));
+                        s[blk][v] = see ? s[blk][v] : WA_NEG;
+                    }
+            }
         }
         float tm = s[0][0];
 #pragma unroll
@@ -429,25 +459,33 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
         }
         const float ref = m > 0.5f * WA_NEG ? m : 0.0f;    // a row that has seen nothing: its scores give exp2(-huge) = 0
         const float sc = a.scale_log2;
+        // the exponentials of the next 16 keys run between the MFMAs of these
+        hy_u32x4 hi[2], lo[2];
+        auto weigh = [&](int st_, int x) __attribute__((always_inline)) {
+            const int v = (st_ & 1) * 8 + 2 * x;
+            const float p0 = __builtin_amdgcn_exp2f(fmaf(s[st_ >> 1][v], sc, -ref)), p1 = __builtin_amdgcn_exp2f(fmaf(s[st_ >> 1][v + 1], sc, -ref));
+            l += p0 + p1;
+            uint32_t tw[2];
+            split2<2>(p0, p1, tw);
+            hi[st_ & 1][x] = tw[0]; lo[st_ & 1][x] = tw[1];
+        };
 #pragma unroll
-        for (int blk = 0; blk < 2; ++blk) {
+        for (int x = 0; x < 4; ++x) weigh(0, x);
 #pragma unroll
-            for (int half = 0; half < 2; ++half) {
-                hy_u32x4 hi, lo;
+        for (int st_ = 0; st_ < 4; ++st_) {
 #pragma unroll
-                for (int x = 0; x < 4; ++x) {
-                    const float p0 = __builtin_amdgcn_exp2f(fmaf(s[blk][half * 8 + 2 * x], sc, -ref)), p1 = __builtin_amdgcn_exp2f(fmaf(s[blk][half * 8 + 2 * x + 1], sc, -ref));
-                    l += p0 + p1;
-                    uint32_t tw[2];
-                    split2<2>(p0, p1, tw);
-                    hi[x] = tw[0]; lo[x] = tw[1];
-                }
+            for (int db = 0; db < DB; ++db) {
+                const int x = st_ * DB + db;
+                if (x + AHEAD < 4 * DB) vf[x + AHEAD] = v_frag(off, (x + AHEAD) / DB, (x + AHEAD) % DB);
+                o[db] = mfma32(vf[x], __builtin_bit_cast(hy_bf16x8, hi[st_ & 1]), o[db]);
+                if (st_ < 3 && db < 2) weigh(st_ + 1, db);
+                __builtin_amdgcn_sched_barrier(0);
+            }
 #pragma unroll
-                for (int db = 0; db < DB; ++db) {
-                    const hy_bf16x8 vf = v_frag(off, blk * 2 + half, db);
-                    o[db] = mfma32(vf, __builtin_bit_cast(hy_bf16x8, hi), o[db]);
-                    o[db] = mfma32(vf, __builtin_bit_cast(hy_bf16x8, lo), o[db]);
-                }
+            for (int db = 0; db < DB; ++db) {
+                o[db] = mfma32(vf[st_ * DB + db], __builtin_bit_cast(hy_bf16x8, lo[st_ & 1]), o[db]);
+                if (st_ < 3 && db < 2) weigh(st_ + 1, 2 + db);
+                __builtin_amdgcn_sched_barrier(0);
             }
         }
     }
@@ -464,13 +502,13 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowArgs a) {
             if (a.vec) {
                 if (d < a.Dv) {
                     const float4 gt = ld4(gr + d);
-                    st4(orow + d, make_float4(o[db][4 * c] * inv * sigmoid_f(gt.x), o[db][4 * c + 1] * inv * sigmoid_f(gt.y),
-                                              o[db][4 * c + 2] * inv * sigmoid_f(gt.z), o[db][4 * c + 3] * inv * sigmoid_f(gt.w)));
+                    st4(orow + d, make_float4(o[db][4 * c] * inv * sigmoid_fast(gt.x), o[db][4 * c + 1] * inv * sigmoid_fast(gt.y),
+                                              o[db][4 * c + 2] * inv * sigmoid_fast(gt.z), o[db][4 * c + 3] * inv * sigmoid_fast(gt.w)));
                 }
             } else {
 #pragma unroll
                 for (int x = 0; x < 4; ++x)
-                    if (d + x < a.Dv) st(orow + d + x, o[db][4 * c + x] * inv * sigmoid_f(ld(gr + d + x)));
+                    if (d + x < a.Dv) st(orow + d + x, o[db][4 * c + x] * inv * sigmoid_fast(ld(gr + d + x)));
             }
         }
     }

@@ -183,7 +183,7 @@ def mlstm(proj: torch.Tensor, offsets: Sequence[int], gates: torch.Tensor, i_bia
     lib, st, code = _lib.load_hybrid(), _lib.current_stream(proj.device), _lib.dtype_code(proj.dtype)
     T, s = proj.shape[0], spec
     qo, ko, vo, go = offsets
-    o = torch.empty(T, s.heads, s.vdim, dtype=torch.float32, device=proj.device)
+    o = torch.empty(T, s.heads, s.vdim, dtype=proj.dtype, device=proj.device)
     out = torch.empty(T, s.heads * s.vdim, dtype=proj.dtype, device=proj.device)
     need = lib.trimkv_mlstm_workspace(batch.batch, batch.max_len, s.heads, s.dim, s.vdim, code)
     ws = torch.empty(need, dtype=torch.float32, device=proj.device) if need else None
