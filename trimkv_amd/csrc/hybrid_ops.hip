@@ -60,18 +60,29 @@ __global__ __launch_bounds__(WAVES * 64) void linear_f32_mfma_kernel(const float
     hy_f32x4 acc[NT];
 #pragma unroll
     for (int j = 0; j < NT; ++j) acc[j] = {0.f, 0.f, 0.f, 0.f};
-    for (int i = wv * 32; i < k; i += WAVES * 32) {     // k is a multiple of 32
-        const float4 a = *(const float4*)(xr + i + kg * 8), b = *(const float4*)(xr + i + kg * 8 + 4);
-        hy_bf16x8 wf[NT];
+    constexpr int UN = NT == 1 ? 4 : 2;                 // k-steps whose operands are requested together
+    for (int i0 = wv * 32; i0 < k; i0 += UN * WAVES * 32) {     // k is a multiple of 32
+        float4 a[UN], b[UN];
+        hy_u32x4 wf[UN][NT];
 #pragma unroll
-        for (int j = 0; j < NT; ++j) wf[j] = *(const hy_bf16x8*)(wr[j] + i + kg * 8);
-        uint32_t s0[3], s1[3], s2[3], s3[3];
-        split2<3>(a.x, a.y, s0); split2<3>(a.z, a.w, s1); split2<3>(b.x, b.y, s2); split2<3>(b.z, b.w, s3);
+        for (int u = 0; u < UN; ++u) {
+            const int i = min(i0 + u * WAVES * 32, k - 32) + kg * 8;
+            a[u] = *(const float4*)(xr + i);
+            b[u] = *(const float4*)(xr + i + 4);
 #pragma unroll
-        for (int e = 2; e >= 0; --e) {
-            const hy_bf16x8 xf = __builtin_bit_cast(hy_bf16x8, (hy_u32x4){s0[e], s1[e], s2[e], s3[e]});
+            for (int j = 0; j < NT; ++j) wf[u][j] = *(const hy_u32x4*)(wr[j] + i);
+        }
 #pragma unroll
-            for (int j = 0; j < NT; ++j) acc[j] = mfma16(xf, wf[j], acc[j]);
+        for (int u = 0; u < UN; ++u) {
+            if (i0 + u * WAVES * 32 >= k) break;
+            uint32_t s0[3], s1[3], s2[3], s3[3];
+            split2<3>(a[u].x, a[u].y, s0); split2<3>(a[u].z, a[u].w, s1); split2<3>(b[u].x, b[u].y, s2); split2<3>(b[u].z, b[u].w, s3);
+#pragma unroll
+            for (int e = 2; e >= 0; --e) {
+                const hy_bf16x8 xf = __builtin_bit_cast(hy_bf16x8, (hy_u32x4){s0[e], s1[e], s2[e], s3[e]});
+#pragma unroll
+                for (int j = 0; j < NT; ++j) acc[j] = mfma16(xf, __builtin_bit_cast(hy_bf16x8, wf[u][j]), acc[j]);
+            }
         }
     }
 #pragma unroll

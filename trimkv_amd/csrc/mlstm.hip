@@ -46,6 +46,22 @@ __global__ __launch_bounds__(256) void mlstm_recurrent_kernel(MlstmArgs a) {
     const float* nm_in = a.nm + parity * copy + at;
     float* nm_out = a.nm + (1 - parity) * copy + at;
     float* Sp = a.S + (((int64_t)slot * a.H + h) * a.D + d0) * a.Dv + (cin ? col : 0);
+    // a token's operands are requested one token ahead (the first ones before the state)
+    float q_next[2], k_next[2], v_next, zi, zf;
+    auto fetch = [&](int t) __attribute__((always_inline)) {
+        const int64_t tok = t0 + min(t, len - 1);
+        const T* row = (const T*)a.p + tok * a.p_stride;
+#pragma unroll
+        for (int x = 0; x < 2; ++x) {
+            const int d = min(tid + 256 * x, a.D - 1);
+            q_next[x] = ld(row + a.q_off + h * a.D + d);
+            k_next[x] = ld(row + a.k_off + h * a.D + d);
+        }
+        v_next = ld(row + a.v_off + h * a.Dv + (cin ? col : 0));
+        zi = a.gates[tok * 2 * a.H + h];
+        zf = a.gates[tok * 2 * a.H + a.H + h];
+    };
+    fetch(0);
     float s[KMAX];
 #pragma unroll
     for (int x = 0; x < KMAX; ++x) s[x] = fresh || x >= nd ? 0.0f : Sp[(int64_t)x * a.Dv];
@@ -54,20 +70,22 @@ __global__ __launch_bounds__(256) void mlstm_recurrent_kernel(MlstmArgs a) {
     const float ib = a.ib[h], fb = a.fb[h];
     for (int t = 0; t < len; ++t) {
         const int64_t tok = t0 + t;
-        const T* row = (const T*)a.p + tok * a.p_stride;
-        const float li = log_input_gate(a.gates[tok * 2 * a.H + h] + ib, a.cap);
-        const float lf = log_forget_gate(a.gates[tok * 2 * a.H + a.H + h] + fb, a.cap);
-        const float v = ld(row + a.v_off + h * a.Dv + (cin ? col : 0));
+        const float li = log_input_gate(zi + ib, a.cap), lf = log_forget_gate(zf + fb, a.cap), v = v_next;
         const float mn = fmaxf(lf + m, li), keep = expf(lf + m - mn), add = expf(li - mn);
         m = mn;
         float qn = 0.0f;
-        for (int d = tid; d < a.D; d += 256) {
-            const float qq = ld(row + a.q_off + h * a.D + d) * a.qscale, kk = ld(row + a.k_off + h * a.D + d);
-            q[d] = qq; k[d] = kk;
-            const float nn = keep * n[d] + add * kk;
-            n[d] = nn;
-            qn += nn * qq;
+#pragma unroll
+        for (int x = 0; x < 2; ++x) {
+            const int d = tid + 256 * x;
+            if (d < a.D) {
+                const float qq = q_next[x] * a.qscale, kk = k_next[x];
+                q[d] = qq; k[d] = kk;
+                const float nn = keep * n[d] + add * kk;
+                n[d] = nn;
+                qn += nn * qq;
+            }
         }
+        if (t + 1 < len) fetch(t + 1);
         qn = block_sum_f(qn, part, 4);            // its barrier also publishes q and k
         const float av = add * v;
         float num = 0.0f;

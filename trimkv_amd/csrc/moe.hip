@@ -17,6 +17,8 @@ namespace trimkv {
 
 constexpr int ROUTE_MAX_E = 1024;
 
+// NE: 64-expert slices, rounded up
+template <int NE>
 __global__ __launch_bounds__(256) void route_kernel(const float* z, const float* correction, int32_t* ids, float* weights, int tokens, int E, int top, int count, int keep) {
     extern __shared__ float rt[];                 // per wavefront: choice [E], group [count]
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -37,9 +39,9 @@ __global__ __launch_bounds__(256) void route_kernel(const float* z, const float*
         group[g] = per > 1 ? a + b : a;
     }
     __syncthreads();
-    float c[ROUTE_MAX_E / 64];
+    float c[NE];
 #pragma unroll
-    for (int i = 0; i < ROUTE_MAX_E / 64; ++i) {
+    for (int i = 0; i < NE; ++i) {
         const int e = i * 64 + lane;
         c[i] = -INFINITY;
         if (e < E) {
@@ -53,7 +55,7 @@ __global__ __launch_bounds__(256) void route_kernel(const float* z, const float*
         float best = -INFINITY;
         int at = 0x7fffffff;
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_E / 64; ++i)
+        for (int i = 0; i < NE; ++i)
             if (c[i] > best) { best = c[i]; at = i * 64 + lane; }
 #pragma unroll
         for (int d = 32; d > 0; d >>= 1) {
@@ -63,7 +65,7 @@ __global__ __launch_bounds__(256) void route_kernel(const float* z, const float*
         }
         at = min(at, E - 1);                      // non-finite logits: stay in bounds
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_E / 64; ++i)
+        for (int i = 0; i < NE; ++i)
             if (i * 64 + lane == at) c[i] = -INFINITY;
         if (live && lane == 0) {
             ids[(int64_t)t * top + j] = at;
@@ -329,8 +331,14 @@ extern "C" int trimkv_moe_route(const float* logits, const float* correction, in
     if (tokens <= 0 || experts <= 0 || experts > ROUTE_MAX_E || groups <= 0 || experts % groups || keep_groups < 1 || keep_groups > groups || top < 1 ||
         top > keep_groups * (experts / groups))
         return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d experts=%d top=%d groups=%d keep=%d", fn, tokens, experts, top, groups, keep_groups);
-    hipLaunchKernelGGL(route_kernel, dim3((tokens + 3) / 4), dim3(256), 4 * (experts + groups) * sizeof(float), (hipStream_t)stream, logits, correction, ids, weights,
-                       tokens, experts, top, groups, keep_groups);
+    auto go = [&](auto ne) {
+        hipLaunchKernelGGL((route_kernel<decltype(ne)::value>), dim3((tokens + 3) / 4), dim3(256), 4 * (experts + groups) * sizeof(float), (hipStream_t)stream,
+                           logits, correction, ids, weights, tokens, experts, top, groups, keep_groups);
+    };
+    if (experts <= 64) go(std::integral_constant<int, 1>{});
+    else if (experts <= 128) go(std::integral_constant<int, 2>{});
+    else if (experts <= 256) go(std::integral_constant<int, 4>{});
+    else go(std::integral_constant<int, ROUTE_MAX_E / 64>{});
     return launch_status(fn);
 }
 

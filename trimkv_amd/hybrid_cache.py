@@ -49,8 +49,7 @@ class HybridCache(_CacheBase):
             for name, (shape, dtype) in spec.state_shapes(num_slots, self.dtype).items():
                 new = torch.zeros(shape, dtype=dtype, device=self.device)
                 if old:
-                    axis = list(shape).index(num_slots) if name != "nm" else 1
-                    new.narrow(axis, 0, old).copy_(state[name])
+                    new.narrow(1 if name == "nm" else 0, 0, old).copy_(state[name])
                 state[name] = new
         seen = torch.zeros(num_slots, 2, dtype=torch.int32, device=self.device)
         seen[:old] = self.seen
