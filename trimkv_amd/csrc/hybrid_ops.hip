@@ -60,7 +60,7 @@ __global__ __launch_bounds__(WAVES * 64) void linear_f32_mfma_kernel(const float
     hy_f32x4 acc[NT];
 #pragma unroll
     for (int j = 0; j < NT; ++j) acc[j] = {0.f, 0.f, 0.f, 0.f};
-    constexpr int UN = NT == 1 ? 4 : 2;                 // k-steps whose operands are requested together
+    constexpr int UN = NT == 1 ? 4 : 1;                 // k-steps whose operands are requested together
     for (int i0 = wv * 32; i0 < k; i0 += UN * WAVES * 32) {     // k is a multiple of 32
         float4 a[UN], b[UN];
         hy_u32x4 wf[UN][NT];
