@@ -20,7 +20,7 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 CONFIGS = {
     "mixed": config([attention(mlp=moe()), mlstm(mlp=moe(experts=8, top=3, ff=24, count=2, keep=1)), mlstm(), attention(heads=2, kv_heads=2, dim=16, vdim=16, size=20, keep_first=0, mlp=moe())]),
-    "recurrent_first": config([mlstm(heads=1, dim=64, vdim=64, gate_cap=15.0, mlp=moe(experts=4, top=1, ff=8, count=1, keep=1)), attention(heads=6, kv_heads=1, dim=48, vdim=64, size=33, keep_first=65, mlp=None)],
+    "recurrent_first": config([mlstm(heads=1, dim=64, vdim=64, gate_cap=15.0, mlp=moe(experts=4, top=1, ff=8, count=1, keep=1)), attention(heads=5, kv_heads=1, dim=48, vdim=56, size=33, keep_first=65, mlp=None)],
                               vocab=130, width=128, eps=1e-6, scale=1.0),
     "attention_only": config([attention(heads=8, kv_heads=4, dim=64, vdim=32, size=70, keep_first=1)], vocab=51, width=200),
     "recurrent_only": config([mlstm(heads=5, dim=20, vdim=12)], vocab=33, width=60),

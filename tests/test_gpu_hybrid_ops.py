@@ -34,7 +34,7 @@ def test_embedding_scale_and_padding(dtype, width):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("rows,n,k", [(1, 3, 64), (17, 40, 320), (70, 16, 1024), (2100, 33, 192), (2050, 130, 128)])
+@pytest.mark.parametrize("rows,n,k", [(1, 3, 64), (17, 40, 352), (70, 16, 1024), (2100, 33, 192), (2050, 130, 128)])
 def test_linear_keeps_fp32(dtype, rows, n, k):
     x, w = rnd(rows, k, seed=1) * 3.0, rnd(n, k, seed=2, dtype=dtype)
     out = ops.linear_f32(x.to(DEV), w.to(DEV))
@@ -238,7 +238,7 @@ def test_mlstm_extreme_gates(dtype, gate_scale, f_shift):
 
 
 # ---- routed experts --------------------------------------------------------------------------------------
-@pytest.mark.parametrize("E,top,count,keep", [(12, 3, 2, 1), (8, 2, 1, 1), (6, 2, 6, 2), (64, 8, 8, 4), (130, 7, 10, 3), (4, 4, 2, 2), (5, 1, 1, 1)])
+@pytest.mark.parametrize("E,top,count,keep", [(14, 3, 2, 1), (8, 2, 1, 1), (6, 2, 6, 2), (64, 8, 8, 4), (130, 7, 10, 3), (4, 4, 2, 2), (5, 1, 1, 1)])
 def test_router(E, top, count, keep):
     z = rnd(300, E, seed=E) * 2
     for shift in (0.0, -3.0):              # all choice scores negative: a closed group must not win with a zero
@@ -250,7 +250,7 @@ def test_router(E, top, count, keep):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,E,top,ff,width", [(1, 6, 2, 40, 72), (5, 3, 1, 64, 64), (37, 12, 3, 24, 100), (700, 8, 3, 136, 200), (130, 4, 4, 320, 256), (900, 5, 2, 64, 520)])
+@pytest.mark.parametrize("T,E,top,ff,width", [(1, 6, 2, 40, 72), (5, 3, 1, 64, 64), (37, 10, 3, 24, 100), (700, 8, 3, 136, 200), (130, 4, 4, 320, 256), (900, 5, 2, 64, 520)])
 def test_experts(dtype, T, E, top, ff, width):
     wp, fp = ops.padded(width), ops.padded(ff)
     x = torch.zeros(T, wp)
