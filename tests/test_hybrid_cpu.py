@@ -1,4 +1,4 @@
-"""CPU checks of the hybrid decoders: ABI of libtrimkv_hybrid.so, configuration and registry, loading, refusal to run without a
+"""CPU checks of the hybrid decoders: ABI of their libraries, configuration and registry, loading, refusal to run without a
 GPU, and the oracle's own mechanisms on cases small enough to work out by hand."""
 import ctypes
 import json
@@ -22,9 +22,8 @@ TEXT = re.sub(r"/\*.*?\*/", "", open(os.path.join(ROOT, "include", "trimkv_hybri
 
 def test_header_binding_and_library_agree():
     declared = sorted(set(re.findall(r"\b(trimkv_[a-z0-9_]+)\s*\(", TEXT)))
-    assert sorted(_lib.HYBRID_SIGNATURES) == declared
-    lib = ctypes.CDLL(_lib.HYBRID_LIB_PATH)
-    for name, (_, argtypes) in _lib.HYBRID_SIGNATURES.items():
+    assert sorted(n for sig in _lib.HYBRID_SIGNATURES.values() for n in sig) == declared
+    for lib, name, argtypes in ((ctypes.CDLL(_lib.HYBRID_LIB_PATHS[l]), n, a) for l, sig in _lib.HYBRID_SIGNATURES.items() for n, (_, a) in sig.items()):
         assert hasattr(lib, name), name
         params = re.search(r"\b%s\s*\(([^;]*?)\)\s*;" % name, TEXT, flags=re.S).group(1).strip()
         want = [] if params in ("", "void") else [p.strip() for p in params.split(",")]
@@ -35,19 +34,25 @@ def test_header_binding_and_library_agree():
 def test_bad_arguments_are_refused_without_a_launch():
     lib = _lib.load_hybrid()
     one = ctypes.c_void_p(16)
-    assert lib.trimkv_embed_scaled(None, one, 1.0, one, None, 1, 4, 8, 64, _lib.F32, None) == -1
-    assert lib.trimkv_embed_scaled(one, one, 1.0, one, None, 1, 4, 8, 64, _lib.F16, None) == -3
+    embed = lambda ids=one, xh=None, norm=None, dt=_lib.F32: lib.trimkv_embed_scaled(ids, one, 1.0, one, xh, norm, 1e-6, 0, 1, 4, 8, 64, dt, None)
+    assert embed(ids=None) == -1 and embed(norm=one) == -1 and embed(dt=_lib.F16) == -3
+    assert lib.trimkv_residual_norm(one, 64, None, 1, one, one, 1.0, None, one, 1, 64, 64, 1e-6, _lib.BF16, None) == -1      # a norm with nowhere to go
+    heads = lambda H=4, D=16, rot=8, table=one, kw=one: lib.trimkv_qkv_heads(one, 256, 0, 64, 80, None, one, kw, 1e-6, table, rot, H, 1, D, D, D, D, one, one, one, None, None, 0, 0, 1, _lib.BF16, None)
+    assert heads(H=0) == -2 and heads(rot=18) == -2 and heads(rot=7) == -2 and heads(table=None) == -1 and heads(kw=None) == -1
+    assert lib.trimkv_rotary_table(one, one, one, one, one, 1, 1, 7, None) == -2 and lib.trimkv_rotary_table(None, one, one, one, one, 1, 1, 8, None) == -1
+    assert lib.trimkv_silu_gate(one, one, 4, one, 1, 8, _lib.BF16, None) == -2 and lib.trimkv_soft_cap(one, one, 4, 0.0, _lib.BF16, None) == -2
     assert lib.trimkv_linear_f32(one, 64, one, 64, one, 1, 3, 62, _lib.F32, None) == -2
     assert b"bad sizes" in lib.trimkv_hybrid_last_error()
-    win = lambda H=4, G=2, D=16, Dp=16, keep=1, size=4, dt=_lib.BF16: lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, H, G, D, D, Dp, Dp, keep, size, 1.0, 1, None, dt, None)
+    win = lambda H=4, G=2, D=16, Dp=16, keep=1, size=4, dt=_lib.BF16: lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, H, G, D, D, Dp, Dp, keep, size, 1.0, 0, 0, 1, None, dt, None)
     assert win(H=5) == -2 and win(Dp=12, D=12) == -2 and win(size=0) == -2 and win(keep=-1) == -2 and win(D=520, Dp=520) == -6 and win(dt=7) == -3
-    assert lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, 4, 2, 16, 16, 16, 16, 1, 4, 1.0, 3, None, _lib.BF16, None) == -5
-    assert lib.trimkv_moe_route(one, one, one, one, 1, 8, 5, 2, 1, None) == -2          # one open group of four cannot give five
-    assert lib.trimkv_moe_route(one, one, one, one, 1, 9, 2, 2, 1, None) == -2
-    assert lib.trimkv_moe_gemm(one, 64, one, one, 64, one, one, one, 4, 2, 16, 1, 64, 64, 64, 1, _lib.BF16, None) == -2
-    assert lib.trimkv_mlstm(one, 64, 0, 8, 16, one, one, one, 1.0, one, one, one, one, one, one, 1, 1, 1, 513, 8, 1, 1.0, None, _lib.F32, None) == -6
+    assert lib.trimkv_window_decode(one, one, one, one, one, one, 64, one, 1, 4, 2, 16, 16, 16, 16, 1, 4, 1.0, 0, 0, 3, None, _lib.BF16, None) == -5
+    recurrent, routed = _lib.load_hybrid("mlstm"), _lib.load_hybrid("moe")
+    assert routed.trimkv_moe_route(one, one, one, one, 1, 8, 5, 2, 1, None) == -2          # one open group of four cannot give five
+    assert routed.trimkv_moe_route(one, one, one, one, 1, 9, 2, 2, 1, None) == -2
+    assert routed.trimkv_moe_gemm(one, 64, one, one, 64, one, one, one, 4, 2, 16, 1, 64, 64, 64, 1, _lib.BF16, None) == -2
+    assert recurrent.trimkv_mlstm(one, 64, 0, 8, 16, one, one, one, 1.0, one, one, one, one, one, one, 1, 1, 1, 513, 8, 1, 1.0, None, _lib.F32, None) == -6
     assert lib.trimkv_window_decode_splits(64, 8, 4096) >= 1 and lib.trimkv_window_decode_splits(1, 1, 64) == 1
-    assert lib.trimkv_mlstm_workspace(1, 1, 4, 64, 64, _lib.BF16) == 0
+    assert recurrent.trimkv_mlstm_workspace(1, 1, 4, 64, 64, _lib.BF16) == 0
 
 
 GOOD = config([attention(mlp=moe()), mlstm()])

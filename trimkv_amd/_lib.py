@@ -10,7 +10,7 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libtrimkv_hip.so")
-HYBRID_LIB_PATH = os.path.join(_HERE, "libtrimkv_hybrid.so")
+HYBRID_LIB_PATHS = {name: os.path.join(_HERE, f"libtrimkv_{name}.so") for name in ("hybrid", "mlstm", "moe")}
 
 F32, BF16, F16 = 0, 1, 2
 SCORE_ALPHA, SCORE_KNORM_ALPHA = 0, 1
@@ -82,29 +82,41 @@ SIGNATURES = {
     "trimkv_stream_probe": (_i, [_p, _p, _i64, _i, _p, _p]),
 }
 
-# the same for trimkv_hybrid.h
+# the same for trimkv_hybrid.h, by library
 HYBRID_SIGNATURES = {
-    "trimkv_hybrid_last_error": (C.c_char_p, []),
-    "trimkv_embed_scaled": (_i, [_p, _p, _f, _p, _p, _i, _i, _i, _i, _i, _p]),
-    "trimkv_linear_f32": (_i, [_p, _i64, _p, _i64, _p, _i, _i, _i, _i, _p]),
-    "trimkv_residual_norm": (_i, [_p, _i64, _p, _i, _p, _p, _p, _i, _i, _i, _f, _i, _p]),
-    "trimkv_rms_rows": (_i, [_p, _i, _p, _p, _p, _i, _i, _f, _i, _p]),
-    "trimkv_qkv_norm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _f, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _p]),
-    "trimkv_ring_store": (_i, [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
-    "trimkv_window_prefill": (_i, [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
-    "trimkv_window_decode_splits": (_i, [_i, _i, _i]),
-    "trimkv_window_decode": (_i, [_p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p, _i, _p]),
-    "trimkv_mlstm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _f, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _p, _i, _p]),
-    "trimkv_mlstm_workspace": (_i64, [_i, _i, _i, _i, _i, _i]),
-    "trimkv_head_norm_gate": (_i, [_p, _p, _i64, _p, _p, _i, _i, _i, _f, _i, _p]),
-    "trimkv_advance": (_i, [_p, _p, _p, _i, _p]),
-    "trimkv_moe_route": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _i, _p]),
-    "trimkv_moe_plan": (_i, [_p, _i, _i, _i, _p, _p, _p, _p]),
-    "trimkv_moe_gemm": (_i, [_p, _i64, _p, _p, _i64, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
+    "hybrid": {
+        "trimkv_hybrid_last_error": (C.c_char_p, []),
+        "trimkv_embed_scaled": (_i, [_p, _p, _f, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _p]),
+        "trimkv_linear_f32": (_i, [_p, _i64, _p, _i64, _p, _i, _i, _i, _i, _p]),
+        "trimkv_residual_norm": (_i, [_p, _i64, _p, _i, _p, _p, _f, _p, _p, _i, _i, _i, _f, _i, _p]),
+        "trimkv_rms_rows": (_i, [_p, _i, _p, _p, _p, _i, _i, _f, _i, _p]),
+        "trimkv_qkv_norm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _f, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _p]),
+        "trimkv_rotary_table": (_i, [_p, _p, _p, _p, _p, _i, _i, _i, _p]),
+        "trimkv_qkv_heads": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _f, _p, _i, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _p]),
+        "trimkv_silu_gate": (_i, [_p, _p, _i64, _p, _i, _i, _i, _p]),
+        "trimkv_soft_cap": (_i, [_p, _p, _i64, _f, _i, _p]),
+        "trimkv_ring_store": (_i, [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
+        "trimkv_window_prefill": (_i, [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p]),
+        "trimkv_window_decode_splits": (_i, [_i, _i, _i]),
+        "trimkv_window_decode": (_i, [_p, _p, _p, _p, _p, _p, _i64, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p, _i, _p]),
+        "trimkv_head_norm_gate": (_i, [_p, _p, _i64, _p, _p, _i, _i, _i, _f, _i, _p]),
+        "trimkv_advance": (_i, [_p, _p, _p, _i, _p]),
+    },
+    "mlstm": {
+        "trimkv_mlstm_last_error": (C.c_char_p, []),
+        "trimkv_mlstm": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _f, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _p, _i, _p]),
+        "trimkv_mlstm_workspace": (_i64, [_i, _i, _i, _i, _i, _i]),
+    },
+    "moe": {
+        "trimkv_moe_last_error": (C.c_char_p, []),
+        "trimkv_moe_route": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _i, _p]),
+        "trimkv_moe_plan": (_i, [_p, _i, _i, _i, _p, _p, _p, _p]),
+        "trimkv_moe_gemm": (_i, [_p, _i64, _p, _p, _i64, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
+    },
 }
 
 _lib = None
-_hybrid = None
+_hybrid = {}
 
 
 def load():
@@ -125,27 +137,27 @@ def load():
     return lib
 
 
-def load_hybrid():
-    """The ctypes handle of libtrimkv_hybrid.so (loaded once); raises if the library has not been built."""
-    global _hybrid
-    if _hybrid is not None:
-        return _hybrid
-    if not os.path.exists(HYBRID_LIB_PATH):
+def load_hybrid(name: str = "hybrid"):
+    """The ctypes handle of one of the hybrid decoders' libraries (loaded once); raises if it has not been built."""
+    if name in _hybrid:
+        return _hybrid[name]
+    path = HYBRID_LIB_PATHS[name]
+    if not os.path.exists(path):
         raise TrimKVLibraryError(
-            f"{HYBRID_LIB_PATH} is missing: build it with `python -m trimkv_amd.build hybrid` (hipcc, gfx950). "
+            f"{path} is missing: build it with `python -m trimkv_amd.build {name}` (hipcc, gfx950). "
             "There is no CPU fallback.")
-    lib = C.CDLL(HYBRID_LIB_PATH)
-    for name, (res, args) in HYBRID_SIGNATURES.items():
-        fn = getattr(lib, name)
+    lib = C.CDLL(path)
+    for fn_name, (res, args) in HYBRID_SIGNATURES[name].items():
+        fn = getattr(lib, fn_name)
         fn.restype = res
         fn.argtypes = args
-    _hybrid = lib
+    _hybrid[name] = lib
     return lib
 
 
-def check_hybrid(rc: int, what: str) -> None:
+def check_hybrid(rc: int, what: str, name: str = "hybrid") -> None:
     if rc != 0:
-        msg = load_hybrid().trimkv_hybrid_last_error().decode("utf-8", "replace")
+        msg = getattr(load_hybrid(name), f"trimkv_{name}_last_error")().decode("utf-8", "replace")
         raise TrimKVLibraryError(f"{what} failed with status {rc}: {msg}")
 
 

@@ -1,8 +1,9 @@
-"""Build the C-ABI libraries of HIP kernels in-tree for gfx950: libtrimkv_hip.so (the TRIM-KV cache path and its decoders)
-and libtrimkv_hybrid.so (decoders with windowed attention, recurrent layers and routed experts).
+"""Build the C-ABI libraries of HIP kernels in-tree for gfx950: libtrimkv_hip.so (the TRIM-KV cache path and its decoders),
+libtrimkv_hybrid.so (what the hybrid decoders share, windowed attention), libtrimkv_mlstm.so and libtrimkv_moe.so (their
+recurrent layers and routed experts).
 
-Usage: ``python -m trimkv_amd.build [--changed] [hip|hybrid ...]`` (hipcc cross-compiles without a GPU; ``--changed``
-recompiles only the sources whose object file is older than its inputs; no name: both libraries).
+Usage: ``python -m trimkv_amd.build [--changed] [hip|hybrid|mlstm|moe ...]`` (hipcc cross-compiles without a GPU; ``--changed``
+recompiles only the sources whose object file is older than its inputs; no name: all of them).
 """
 from __future__ import annotations
 
@@ -15,10 +16,10 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 INCLUDE = os.path.join(os.path.dirname(HERE), "include")
 LIB_PATH = os.path.join(HERE, "libtrimkv_hip.so")
-HYBRID_LIB_PATH = os.path.join(HERE, "libtrimkv_hybrid.so")
 SOURCES = ["api.hip", "append.hip", "evict.hip", "attn_decode.hip", "attn_decode_append.hip", "attn_decode_pieces.hip", "attn_decode_append_pieces.hip", "attn_decode_append_gated.hip", "attn_decode_append_pieces_gated.hip", "pieces_plan.hip", "attn_prefill.hip", "gate.hip", "stream_probe.hip", "decoder_ops.hip"]
-HYBRID_SOURCES = ["hybrid_ops.hip", "window_attn.hip", "mlstm.hip", "moe.hip"]
-LIBRARIES = {"hip": (LIB_PATH, SOURCES), "hybrid": (HYBRID_LIB_PATH, HYBRID_SOURCES)}
+HYBRID_SOURCES = ["hybrid_ops.hip", "window_attn.hip"]
+LIBRARIES = {"hip": (LIB_PATH, SOURCES), "hybrid": (os.path.join(HERE, "libtrimkv_hybrid.so"), HYBRID_SOURCES),
+             "mlstm": (os.path.join(HERE, "libtrimkv_mlstm.so"), ["mlstm.hip"]), "moe": (os.path.join(HERE, "libtrimkv_moe.so"), ["moe.hip"])}
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-I" + INCLUDE, "-I" + CSRC,
@@ -45,7 +46,7 @@ def _stale(src: str, obj: str) -> bool:
     return any(os.path.getmtime(d) > os.path.getmtime(obj) for d in deps)
 
 
-def build(verbose: bool = True, only_changed: bool = False, libraries=("hip", "hybrid")) -> str:
+def build(verbose: bool = True, only_changed: bool = False, libraries=tuple(LIBRARIES)) -> str:
     """Compile every source of the named libraries (or, with ``only_changed``, the ones whose object is older than its
     inputs) and link them."""
     hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
@@ -74,7 +75,14 @@ def build(verbose: bool = True, only_changed: bool = False, libraries=("hip", "h
     return LIBRARIES[libraries[-1]][0]
 
 
+def ensure(libraries) -> None:
+    """Build those of the named libraries that are not there (a fresh checkout)."""
+    missing = tuple(n for n in libraries if not os.path.exists(LIBRARIES[n][0]))
+    if missing:
+        build(verbose=False, only_changed=True, libraries=missing)
+
+
 if __name__ == "__main__":
     names = [a for a in sys.argv[1:] if not a.startswith("--")]
-    build(only_changed="--changed" in sys.argv[1:], libraries=tuple(names) or ("hip", "hybrid"))
+    build(only_changed="--changed" in sys.argv[1:], libraries=tuple(names) or tuple(LIBRARIES))
     sys.exit(0)

@@ -1,11 +1,16 @@
 // The row-wise work of the hybrid decoders, one launch each; the residual stream is fp32.
 //
-//   trimkv_embed_scaled    x = table[id] * scale
+//   trimkv_embed_scaled    x = table[id] * scale, or x += ..., optionally normed for the first sublayer
 //   trimkv_linear_f32      fp32 rows times a narrow matrix with fp32 results (routers, gates of a recurrence)
-//   trimkv_residual_norm   x += w * rms(y), y one row or a weighted sum of several (the experts of a token)
+//   trimkv_residual_norm   x += mult * w * rms(y), y one row or a weighted sum of several (the experts of a token); the new x
+//                          or its norm for the next sublayer goes along in the matrices' dtype
 //   trimkv_rms_rows        w * rms(x) of chosen rows
 //   trimkv_qkv_norm        RMS norm over the whole q and the whole k projection; q, k, v into head-major padded rows, or k
 //                          and v straight into the window ring (decode)
+//   trimkv_rotary_table    cosines and sines of a step's positions, once for all layers that turn alike
+//   trimkv_qkv_heads       bias, RMS norm per head and rotary positions; q, k, v go where trimkv_qkv_norm puts them
+//   trimkv_silu_gate       silu(gate) * up
+//   trimkv_soft_cap        cap * tanh(x / cap) in fp32
 //   trimkv_ring_store      the rows of a prompt that outlive it, into the window ring
 //   trimkv_head_norm_gate  per-head RMS norm, weight and sigmoid gate behind a recurrence
 //   trimkv_advance         tokens and steps seen per sequence slot
@@ -15,14 +20,70 @@
 namespace trimkv {
 
 // ---- embedding -------------------------------------------------------------------------------
+struct EmbedArgs {
+    const int64_t* ids; const void* table; float scale;
+    float* x; void* xh; const float* norm_w; float eps;
+    int vocab, width, xs, add;
+};
 template <typename T>
-__global__ __launch_bounds__(256) void embed_kernel(const int64_t* ids, const T* table, float scale, float* x, T* xh, int vocab, int width, int xs) {
+__global__ __launch_bounds__(256) void embed_kernel(EmbedArgs a) {
+    __shared__ float part[4];
     const int64_t t = blockIdx.x;
-    const int64_t id = min(max(ids[t], (int64_t)0), (int64_t)vocab - 1);
-    for (int i = threadIdx.x; i < xs; i += 256) {
-        const float f = i < width ? ld(table + id * width + i) * scale : 0.0f;
-        x[t * xs + i] = f;
-        if (xh) st(xh + t * xs + i, f);
+    const int64_t id = min(max(a.ids[t], (int64_t)0), (int64_t)a.vocab - 1);
+    const T* src = (const T*)a.table + id * a.width;
+    float* xr = a.x + t * a.xs;
+    T* hr = (T*)a.xh + t * a.xs;
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < a.xs; i += 256) {
+        float f = i < a.width ? ld(src + i) * a.scale : 0.0f;
+        if (a.add) f += xr[i];
+        xr[i] = f;
+        ss += f * f;
+        if (a.xh && !a.norm_w) st(hr + i, f);
+    }
+    if (!a.norm_w) return;
+    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+    for (int i = threadIdx.x; i < a.xs; i += 256)        // a thread re-reads what it wrote itself
+        st(hr + i, i < a.width ? xr[i] * inv * a.norm_w[i] : 0.0f);
+}
+// width and stride multiples of 4, width up to 1024 NV: a row stays in registers
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void embed_vec_kernel(EmbedArgs a) {
+    __shared__ float part[4];
+    const int64_t t = blockIdx.x;
+    const int64_t id = min(max(a.ids[t], (int64_t)0), (int64_t)a.vocab - 1);
+    const T* src = (const T*)a.table + id * a.width;
+    float* xr = a.x + t * a.xs;
+    T* hr = (T*)a.xh + t * a.xs;
+    const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+    float4 f[NV];
+    float ss = 0.0f;
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+        const int i = (v * 256 + threadIdx.x) * 4;
+        f[v] = zero;
+        if (i < a.width) {
+            f[v] = ld4(src + i);
+            f[v].x *= a.scale; f[v].y *= a.scale; f[v].z *= a.scale; f[v].w *= a.scale;
+            if (a.add) {
+                const float4 o = *(const float4*)(xr + i);
+                f[v].x += o.x; f[v].y += o.y; f[v].z += o.z; f[v].w += o.w;
+            }
+        }
+        if (i < a.xs) {
+            *(float4*)(xr + i) = f[v];
+            if (a.xh && !a.norm_w) st4(hr + i, f[v]);
+        }
+        ss += f[v].x * f[v].x + f[v].y * f[v].y + f[v].z * f[v].z + f[v].w * f[v].w;
+    }
+    if (!a.norm_w) return;
+    const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+        const int i = (v * 256 + threadIdx.x) * 4;
+        if (i >= a.xs) continue;
+        const float4 w = i < a.width ? *(const float4*)(a.norm_w + i) : zero;
+        st4(hr + i, make_float4(f[v].x * inv * w.x, f[v].y * inv * w.y, f[v].z * inv * w.z, f[v].w * inv * w.w));
     }
 }
 
@@ -98,16 +159,17 @@ __global__ __launch_bounds__(WAVES * 64) void linear_f32_mfma_kernel(const float
     }
 }
 
-// ---- residual += w * rms(y) --------------------------------------------------------------------
+// ---- residual += mult * w * rms(y) --------------------------------------------------------------------
 struct ResidualNormArgs {
     const void* y; int64_t y_stride; const float* y_weight; int top;
     float* x; const float* w; void* xh; int width, xs; float eps;
+    float mult; const float* next_w;                  // next_w: xh = next_w * rms(new x) instead of a copy
 };
 // NV > 0: rows of up to 1024 NV elements, four at a time, held in registers; everything is requested before the reduction.
 template <typename T, int NV>
 __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) {
     extern __shared__ float row[];     // NV = 0: width floats, y of this token summed over its experts
-    __shared__ float part[4];
+    __shared__ float part[4], part2[4];
     const int64_t t = blockIdx.x;
     const int tid = threadIdx.x;
     const T* y = (const T*)a.y + t * a.top * a.y_stride;
@@ -140,15 +202,26 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
             }
 #pragma unroll
         for (int v = 0; v < NV; ++v) ss += s[v].x * s[v].x + s[v].y * s[v].y + s[v].z * s[v].z + s[v].w * s[v].w;
-        const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+        const float inv = a.mult / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+        float s2 = 0.0f;
 #pragma unroll
         for (int v = 0; v < NV; ++v) {
             const int i = (v * 256 + tid) * 4;
             if (i < a.width) {
                 f[v].x += s[v].x * inv * w[v].x; f[v].y += s[v].y * inv * w[v].y; f[v].z += s[v].z * inv * w[v].z; f[v].w += s[v].w * inv * w[v].w;
                 *(float4*)(xr + i) = f[v];
-                if (a.xh) st4(hr + i, f[v]);
+                if (a.next_w) {
+                    s2 += f[v].x * f[v].x + f[v].y * f[v].y + f[v].z * f[v].z + f[v].w * f[v].w;
+                    w[v] = *(const float4*)(a.next_w + i);
+                } else if (a.xh) st4(hr + i, f[v]);
             }
+        }
+        if (!a.next_w) return;
+        const float inv2 = 1.0f / sqrtf(block_sum_f(s2, part2, 4) / (float)a.width + a.eps);
+#pragma unroll
+        for (int v = 0; v < NV; ++v) {
+            const int i = (v * 256 + tid) * 4;
+            if (i < a.width) st4(hr + i, make_float4(f[v].x * inv2 * w[v].x, f[v].y * inv2 * w[v].y, f[v].z * inv2 * w[v].z, f[v].w * inv2 * w[v].w));
         }
     } else {
         for (int i = tid; i < a.width; i += 256) {
@@ -158,12 +231,18 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
             row[i] = s;
             ss += s * s;
         }
-        const float inv = 1.0f / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+        const float inv = a.mult / sqrtf(block_sum_f(ss, part, 4) / (float)a.width + a.eps);
+        float s2 = 0.0f;
         for (int i = tid; i < a.width; i += 256) {      // a thread re-reads what it wrote itself
             const float f = xr[i] + row[i] * inv * a.w[i];
             xr[i] = f;
-            if (a.xh) st(hr + i, f);
+            row[i] = f;
+            s2 += f * f;
+            if (a.xh && !a.next_w) st(hr + i, f);
         }
+        if (!a.next_w) return;
+        const float inv2 = 1.0f / sqrtf(block_sum_f(s2, part2, 4) / (float)a.width + a.eps);
+        for (int i = tid; i < a.width; i += 256) st(hr + i, row[i] * inv2 * a.next_w[i]);
     }
 }
 
@@ -293,6 +372,169 @@ __global__ __launch_bounds__(256) void qkv_norm_kernel(QkvNormArgs a) {
     }
 }
 
+// ---- rotary positions, bias and a norm per head ----------------------------------------------------
+// table [tokens][rot]: cosines of the rot / 2 pairs, then their sines.  Angles in fp64: exact positions, and no table of all
+// positions to keep.
+__global__ __launch_bounds__(64) void rotary_table_kernel(const double* freq, const int32_t* cu, const int32_t* slots, const int32_t* seen, float* table, int half) {
+    const int b = blockIdx.y, t0 = cu[b], i = blockIdx.x;
+    if (i >= cu[b + 1] - t0) return;
+    const double pos = (double)(seen[2 * slots[b]] + i);
+    float* row = table + (int64_t)(t0 + i) * 2 * half;
+    for (int j = threadIdx.x; j < half; j += 64) {
+        double s, c;
+        sincos(pos * freq[j], &s, &c);
+        row[j] = (float)c;
+        row[half + j] = (float)s;
+    }
+}
+
+struct QkvHeadsArgs {
+    const void* p; int64_t p_stride; int q_off, k_off, v_off;
+    const float* bias; const float* qw; const float* kw; const float* table;      // each may be absent (the two weights together)
+    float eps;
+    int H, G, D, Dv, Dp, Dvp, rot;
+    void* q; void* k; void* v;
+    const int32_t* slots; const int32_t* seen; int keep, size;
+};
+// where head idx of q (kind 0), k (1) or v (2) of token t goes
+template <typename T>
+__device__ __forceinline__ T* qkv_heads_row(const QkvHeadsArgs& a, int64_t t, int kind, int idx) {
+    if (kind == 0) return (T*)a.q + (t * a.H + idx) * a.Dp;
+    T* base = (T*)(kind == 1 ? a.k : a.v);
+    const int n = kind == 1 ? a.Dp : a.Dvp;
+    if (!a.slots) return base + (t * a.G + idx) * n;
+    const int slot = a.slots[t], cap = a.keep + a.size;
+    return base + (((int64_t)slot * a.G + idx) * cap + ring_slot(a.seen[2 * slot], a.keep, a.size)) * n;
+}
+
+// LH lanes of sixteen values per head: below the rotated size eight values and their eight partners, behind it neighbours.
+// A workgroup keeps to one token, so its lanes' cosines and sines stay in registers over its heads.
+template <typename T, int LH>
+__global__ __launch_bounds__(256) void qkv_heads_vec_kernel(QkvHeadsArgs a) {
+    const int64_t t = blockIdx.x;
+    const int sub = threadIdx.x / LH, l = threadIdx.x % LH, groups = blockDim.x / LH;
+    const int half = a.rot / 2, rl = a.rot / 16, heads = a.H + 2 * a.G;
+    const bool turned = l < rl;
+    const int e0 = turned ? 8 * l : a.rot + 16 * (l - rl), e1 = turned ? half + 8 * l : e0 + 8;
+    const T* row = (const T*)a.p + t * a.p_stride;
+    Eight c, s, w0, w1;
+#pragma unroll
+    for (int x = 0; x < 8; ++x) { c.f[x] = 1.0f; s.f[x] = 0.0f; w0.f[x] = w1.f[x] = 1.0f; }
+    if (turned) {
+        c = ld8(a.table + t * a.rot + 8 * l);
+        s = ld8(a.table + t * a.rot + half + 8 * l);
+    }
+    int held = -1;                                    // whose norm weights w0, w1 hold
+    for (int h = blockIdx.y * groups + sub; h < heads; h += gridDim.y * groups) {
+        const int kind = h < a.H ? 0 : h < a.H + a.G ? 1 : 2;
+        const int idx = kind == 0 ? h : kind == 1 ? h - a.H : h - a.H - a.G;
+        const int n = kind == 2 ? a.Dv : a.D, off = kind == 0 ? a.q_off + idx * a.D : kind == 1 ? a.k_off + idx * a.D : a.v_off + idx * a.Dv;
+        const int i0 = kind == 2 ? 16 * l : e0, i1 = kind == 2 ? 16 * l + 8 : e1;
+        const bool in0 = i0 < n, in1 = i1 < n;
+        Eight x0, x1;
+#pragma unroll
+        for (int x = 0; x < 8; ++x) x0.f[x] = x1.f[x] = 0.0f;
+        if (in0) x0 = ld8(row + off + i0);
+        if (in1) x1 = ld8(row + off + i1);
+        if (a.bias) {
+            if (in0) { const Eight b = ld8(a.bias + off + i0);
+#pragma unroll
+                for (int x = 0; x < 8; ++x) x0.f[x] += b.f[x]; }
+            if (in1) { const Eight b = ld8(a.bias + off + i1);
+#pragma unroll
+                for (int x = 0; x < 8; ++x) x1.f[x] += b.f[x]; }
+        }
+        if (kind < 2) {
+            float inv = 1.0f;
+            if (a.qw) {
+                if (held != kind) {
+                    const float* w = kind ? a.kw : a.qw;
+                    if (in0) w0 = ld8(w + i0);
+                    if (in1) w1 = ld8(w + i1);
+                    held = kind;
+                }
+                float ss = 0.0f;
+#pragma unroll
+                for (int x = 0; x < 8; ++x) ss += x0.f[x] * x0.f[x] + x1.f[x] * x1.f[x];
+#pragma unroll
+                for (int d = LH / 2; d > 0; d >>= 1) ss += __shfl_xor(ss, d, 64);
+                inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+            }
+#pragma unroll
+            for (int x = 0; x < 8; ++x) {
+                const float u = x0.f[x] * inv * w0.f[x], v = x1.f[x] * inv * w1.f[x];
+                x0.f[x] = u * c.f[x] - v * s.f[x];
+                x1.f[x] = v * c.f[x] + u * s.f[x];
+            }
+        }
+        T* dst = qkv_heads_row<T>(a, t, kind, idx);
+        if (in0) st8(dst + i0, x0);
+        if (in1) st8(dst + i1, x1);
+    }
+}
+
+// General form: one wavefront per (token, head), partners read again.
+template <typename T>
+__global__ __launch_bounds__(256) void qkv_heads_kernel(QkvHeadsArgs a, int64_t units) {
+    const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (unit >= units) return;
+    const int heads = a.H + 2 * a.G, lane = threadIdx.x & 63;
+    const int64_t t = unit / heads;
+    const int h = (int)(unit - t * heads);
+    const int kind = h < a.H ? 0 : h < a.H + a.G ? 1 : 2;
+    const int idx = kind == 0 ? h : kind == 1 ? h - a.H : h - a.H - a.G;
+    const int n = kind == 2 ? a.Dv : a.D, off = kind == 0 ? a.q_off + idx * a.D : kind == 1 ? a.k_off + idx * a.D : a.v_off + idx * a.Dv;
+    const T* src = (const T*)a.p + t * a.p_stride + off;
+    const float* w = kind == 0 ? a.qw : kind == 1 ? a.kw : nullptr;
+    const int rot = kind == 2 ? 0 : a.rot, half = rot / 2;
+    float inv = 1.0f;
+    if (w) {
+        float ss = 0.0f;
+        for (int i = lane; i < n; i += 64) { const float f = ld(src + i) + (a.bias ? a.bias[off + i] : 0.0f); ss += f * f; }
+        inv = 1.0f / sqrtf(wave_sum_f(ss) / (float)n + a.eps);
+    }
+    auto value = [&](int i) { return (ld(src + i) + (a.bias ? a.bias[off + i] : 0.0f)) * inv * (w ? w[i] : 1.0f); };
+    T* dst = qkv_heads_row<T>(a, t, kind, idx);
+    for (int i = lane; i < (kind == 2 ? a.Dvp : a.Dp); i += 64) {
+        float f = i < n ? value(i) : 0.0f;
+        if (i < rot) {
+            const int j = i < half ? i : i - half;
+            const float c = a.table[t * rot + j], s = a.table[t * rot + half + j];
+            f = i < half ? f * c - value(i + half) * s : f * c + value(i - half) * s;
+        }
+        st(dst + i, f);
+    }
+}
+
+// ---- silu(gate) * up -----------------------------------------------------------------------------
+__device__ __forceinline__ float silu_gate(const bf16_t*, float g, float u) { return g * sigmoid_fast(g) * u; }
+__device__ __forceinline__ float silu_gate(const float*, float g, float u) { return g * sigmoid_f(g) * u; }
+
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void silu_gate_kernel(const T* gate, const T* up, int64_t stride, T* out, int per_row, int64_t n) {
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+        const int64_t t = i / per_row;
+        const int64_t at = t * stride + (i - t * per_row) * PER;
+        if constexpr (PER == 8) {
+            Eight g = ld8(gate + at);
+            const Eight u = ld8(up + at);
+#pragma unroll
+            for (int x = 0; x < 8; ++x) g.f[x] = silu_gate(out, g.f[x], u.f[x]);
+            st8(out + i * 8, g);
+        } else st(out + i, silu_gate(out, ld(gate + at), ld(up + at)));
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void soft_cap_kernel(const T* x, float* out, int64_t n, float cap) {
+    const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 4;
+    if (i + 4 <= n) {
+        const float4 f = ld4(x + i);
+        *(float4*)(out + i) = make_float4(cap * tanhf(f.x / cap), cap * tanhf(f.y / cap), cap * tanhf(f.z / cap), cap * tanhf(f.w / cap));
+    } else
+        for (int64_t j = i; j < n; ++j) out[j] = cap * tanhf(ld(x + j) / cap);
+}
+
 // ---- a prompt's surviving rows into the ring -----------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void ring_store_kernel(const T* k, const T* v, const int32_t* cu, const int32_t* slots, const int32_t* seen,
@@ -380,13 +622,18 @@ using namespace trimkv;
 
 extern "C" const char* trimkv_hybrid_last_error(void) { return err_buf(); }
 
-extern "C" int trimkv_embed_scaled(const int64_t* ids, const void* table, float scale, float* x, void* xh, int tokens, int vocab, int width,
-                                   int x_stride, int dtype, void* stream) {
+extern "C" int trimkv_embed_scaled(const int64_t* ids, const void* table, float scale, float* x, void* xh, const float* norm_weight, float eps, int add,
+                                   int tokens, int vocab, int width, int x_stride, int dtype, void* stream) {
     const char* fn = "trimkv_embed_scaled";
-    if (!ids || !table || !x) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    if (!ids || !table || !x || (norm_weight && !xh)) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
     HY_CHECK_DTYPE(fn, dtype);
     if (tokens <= 0 || vocab <= 0 || width <= 0 || x_stride < width) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d vocab=%d width=%d stride=%d", fn, tokens, vocab, width, x_stride);
-    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((embed_kernel<T>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, ids, (const T*)table, scale, x, (T*)xh, vocab, width, x_stride));
+    EmbedArgs a{ids, table, scale, x, xh, norm_weight, eps, vocab, width, x_stride, add};
+    const bool vec = width % 4 == 0 && x_stride % 4 == 0 && !(((uintptr_t)table | (uintptr_t)x | (uintptr_t)xh | (uintptr_t)norm_weight) & 15);
+    HY_BY_DTYPE(dtype, T,
+        if (vec && x_stride <= 1024) hipLaunchKernelGGL((embed_vec_kernel<T, 1>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+        else if (vec && x_stride <= 4096) hipLaunchKernelGGL((embed_vec_kernel<T, 4>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+        else hipLaunchKernelGGL((embed_kernel<T>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a));
     return launch_status(fn);
 }
 
@@ -413,16 +660,16 @@ extern "C" int trimkv_linear_f32(const float* x, int64_t x_stride, const void* w
     return launch_status(fn);
 }
 
-extern "C" int trimkv_residual_norm(const void* y, int64_t y_stride, const float* y_weight, int top, float* x, const float* w, void* xh,
-                                    int tokens, int width, int x_stride, float eps, int dtype, void* stream) {
+extern "C" int trimkv_residual_norm(const void* y, int64_t y_stride, const float* y_weight, int top, float* x, const float* w, float mult, void* xh,
+                                    const float* next_w, int tokens, int width, int x_stride, float eps, int dtype, void* stream) {
     const char* fn = "trimkv_residual_norm";
-    if (!y || !x || !w) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    if (!y || !x || !w || (next_w && !xh)) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
     HY_CHECK_DTYPE(fn, dtype);
     if (tokens <= 0 || width <= 0 || width > 16384 || top < 1 || x_stride < width || y_stride < width)
         return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d width=%d top=%d", fn, tokens, width, top);
     if (!y_weight && top != 1) return fail(TRIMKV_ERR_SHAPE, "%s: several rows per token need weights", fn);
-    ResidualNormArgs a{y, y_stride, y_weight, top, x, w, xh, width, x_stride, eps};
-    const bool vec = width % 4 == 0 && x_stride % 4 == 0 && y_stride % 4 == 0 && !((((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)xh)) & 15);
+    ResidualNormArgs a{y, y_stride, y_weight, top, x, w, xh, width, x_stride, eps, mult, next_w};
+    const bool vec = width % 4 == 0 && x_stride % 4 == 0 && y_stride % 4 == 0 && !(((uintptr_t)y | (uintptr_t)x | (uintptr_t)w | (uintptr_t)xh | (uintptr_t)next_w) & 15);
     const size_t lds = (size_t)width * 4;
     HY_BY_DTYPE(dtype, T,
         if (vec && width <= 1024) hipLaunchKernelGGL((residual_norm_kernel<T, 1>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
@@ -458,6 +705,79 @@ extern "C" int trimkv_qkv_norm(const void* proj, int64_t proj_stride, int q_off,
         return launch_status(fn);
     }
     HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((qkv_norm_kernel<T>), dim3(tokens, 2), dim3(256), 0, (hipStream_t)stream, a));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_rotary_table(const double* freq, const int32_t* cu, const int32_t* slots, const int32_t* seen, float* table, int batch, int max_len, int rot_dims, void* stream) {
+    const char* fn = "trimkv_rotary_table";
+    if (!freq || !cu || !slots || !seen || !table) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    if (batch <= 0 || batch > 65535 || max_len <= 0 || rot_dims <= 0 || rot_dims % 2) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes batch=%d max_len=%d rot_dims=%d", fn, batch, max_len, rot_dims);
+    hipLaunchKernelGGL(rotary_table_kernel, dim3(max_len, batch), dim3(64), 0, (hipStream_t)stream, freq, cu, slots, seen, table, rot_dims / 2);
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_qkv_heads(const void* proj, int64_t proj_stride, int q_off, int k_off, int v_off, const float* bias, const float* q_weight, const float* k_weight, float eps,
+                                const float* table, int rot_dims, int heads, int kv_heads, int dim, int vdim, int dim_stride, int vdim_stride, void* q, void* k, void* v,
+                                const int32_t* slots, const int32_t* seen, int keep_first, int window, int tokens, int dtype, void* stream) {
+    const char* fn = "trimkv_qkv_heads";
+    if (!proj || !q || !k || !v || (!slots != !seen) || (!q_weight != !k_weight) || (!table && rot_dims)) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || dim_stride < dim || vdim_stride < vdim || rot_dims < 0 || rot_dims > dim || rot_dims % 2 ||
+        (slots && (window <= 0 || keep_first < 0)))
+        return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d heads=%d kv_heads=%d dim=%d vdim=%d rot_dims=%d", fn, tokens, heads, kv_heads, dim, vdim, rot_dims);
+    QkvHeadsArgs a{proj, proj_stride, q_off, k_off, v_off, bias, q_weight, k_weight, table, eps, heads, kv_heads, dim, vdim, dim_stride, vdim_stride, rot_dims, q, k, v, slots, seen, keep_first, window};
+    hipStream_t s = (hipStream_t)stream;
+    const int units = heads + 2 * kv_heads;
+    const int lanes_qk = rot_dims / 16 + (dim - rot_dims + 15) / 16, lanes_v = (vdim + 15) / 16, lanes = lanes_qk > lanes_v ? lanes_qk : lanes_v;
+    const bool vec = dim_stride == dim && vdim_stride == vdim && dim % 8 == 0 && vdim % 8 == 0 && rot_dims % 16 == 0 && lanes <= 32 && proj_stride % 8 == 0 &&
+                     (q_off | k_off | v_off) % 8 == 0 &&
+                     !(((uintptr_t)proj | (uintptr_t)bias | (uintptr_t)q_weight | (uintptr_t)k_weight | (uintptr_t)table | (uintptr_t)q | (uintptr_t)k | (uintptr_t)v) & 15);
+    if (vec) {
+        auto go = [&](auto lh) {
+            constexpr int LH = decltype(lh)::value;
+            // few tokens: one head per group of lanes; many: a workgroup walks the heads of its token in equal turns
+            int threads = 256, waste = 1 << 30;
+            for (int n = 256; n >= 64; n /= 2) {
+                const int groups = n / LH, idle = (units + groups - 1) / groups * groups - units;
+                if (idle < waste) { waste = idle; threads = n; }
+            }
+            const int groups = threads / LH, spread = tokens < 1024 ? (units + groups - 1) / groups : 1;
+            HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((qkv_heads_vec_kernel<T, LH>), dim3(tokens, spread), dim3(threads), 0, s, a));
+        };
+        if (lanes <= 4) go(std::integral_constant<int, 4>{});
+        else if (lanes <= 8) go(std::integral_constant<int, 8>{});
+        else if (lanes <= 16) go(std::integral_constant<int, 16>{});
+        else go(std::integral_constant<int, 32>{});
+        return launch_status(fn);
+    }
+    const int64_t n = (int64_t)tokens * units;
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((qkv_heads_kernel<T>), dim3((unsigned)((n + 3) / 4)), dim3(256), 0, s, a, n));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_silu_gate(const void* gate, const void* up, int64_t stride, void* out, int tokens, int inter, int dtype, void* stream) {
+    const char* fn = "trimkv_silu_gate";
+    if (!gate || !up || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    if (tokens <= 0 || inter <= 0 || stride < inter) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes tokens=%d inter=%d stride=%lld", fn, tokens, inter, (long long)stride);
+    const bool vec = inter % 8 == 0 && stride % 8 == 0 && !(((uintptr_t)gate | (uintptr_t)up | (uintptr_t)out) & 15);
+    const int per_row = vec ? inter / 8 : inter;
+    const int64_t n = (int64_t)tokens * per_row, blocks = (n + 255) / 256;
+    const dim3 grid((unsigned)(blocks < 65536 ? blocks : 65536));
+    HY_BY_DTYPE(dtype, T,
+        if (vec) hipLaunchKernelGGL((silu_gate_kernel<T, 8>), grid, dim3(256), 0, (hipStream_t)stream, (const T*)gate, (const T*)up, stride, (T*)out, per_row, n);
+        else hipLaunchKernelGGL((silu_gate_kernel<T, 1>), grid, dim3(256), 0, (hipStream_t)stream, (const T*)gate, (const T*)up, stride, (T*)out, per_row, n));
+    return launch_status(fn);
+}
+
+extern "C" int trimkv_soft_cap(const void* x, float* out, int64_t count, float cap, int dtype, void* stream) {
+    const char* fn = "trimkv_soft_cap";
+    if (!x || !out) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
+    HY_CHECK_DTYPE(fn, dtype);
+    const int64_t blocks = (count + 1023) / 1024;
+    if (count <= 0 || blocks > 0x7fffffffLL || !(cap > 0.0f)) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes count=%lld cap=%g", fn, (long long)count, (double)cap);
+    if (((uintptr_t)x | (uintptr_t)out) & 15) return fail(TRIMKV_ERR_SHAPE, "%s: x and out must be 16-byte aligned", fn);
+    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((soft_cap_kernel<T>), dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (const T*)x, out, count, cap));
     return launch_status(fn);
 }
 

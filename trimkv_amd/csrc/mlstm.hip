@@ -522,6 +522,8 @@ static int chunk_segments(int batch, int max_len, int heads, int vdim) {
 
 using namespace trimkv;
 
+extern "C" const char* trimkv_mlstm_last_error(void) { return err_buf(); }
+
 extern "C" int64_t trimkv_mlstm_workspace(int batch, int max_len, int heads, int dim, int vdim, int dtype) {
     if (batch <= 0 || max_len <= 1 || heads <= 0 || dim <= 0 || vdim <= 0 || dtype != TRIMKV_BF16) return 0;
     const int n = chunk_segments(batch, max_len, heads, vdim);

@@ -324,6 +324,8 @@ static int launch_big(const GroupedArgs& a, int most, hipStream_t s) {
 
 using namespace trimkv;
 
+extern "C" const char* trimkv_moe_last_error(void) { return err_buf(); }
+
 extern "C" int trimkv_moe_route(const float* logits, const float* correction, int32_t* ids, float* weights, int tokens, int experts, int top, int groups,
                                 int keep_groups, void* stream) {
     const char* fn = "trimkv_moe_route";

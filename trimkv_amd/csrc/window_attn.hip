@@ -1,6 +1,6 @@
 // Sliding-window attention with kept first tokens over a ring of keys and values -- gfx950.
 //
-// Position i sees j iff j <= i and (i - j < size or j < keep).  Keys carry no position of their own, so a sequence needs
+// Position i sees j iff j <= i and (i - j < size or j < keep).  Keys arrive as they are scored (rotated, if at all), so a sequence needs
 // exactly keep + size rows however long it is: the first `keep` tokens own their rows, later ones overwrite the row of the
 // token that has just left the window.  After a token is stored, the rows in use are its visible set, and the decode kernel
 // walks them in storage order without any mask.
@@ -12,7 +12,8 @@
 //   window_rows_kernel     the same for fp32 and for head sizes beyond the tiles: one wavefront per query
 //
 // Scores, maxima, exponentials and sums are fp32; scores are scaled after the product.  In the prefill kernel the
-// probabilities enter the second product as two bf16 terms each (17 bits).  The sigmoid output gate is applied on the way out.
+// probabilities enter the second product as two bf16 terms each (17 bits).  The sigmoid output gate (a number per value or one
+// per head) is applied on the way out.  With a sink the denominator has one more term, a score of 0 without a value.
 #include "hybrid.hip.h"
 #include <type_traits>
 
@@ -29,7 +30,15 @@ struct WindowArgs {
     float scale_log2;
     int chunk, splits; float* ws;                     // decode: rows per workgroup; partial results
     int vec;                                          // gate and out may be accessed four elements at a time
+    int head_gate;                                    // one gate per head instead of one per value
+    int sink;                                         // the softmax denominator starts at exp(0)
 };
+template <typename T>
+__device__ __forceinline__ float window_gate(const WindowArgs& a, int64_t t, int h, int d) {
+    return sigmoid_fast(ld((const T*)a.gate + t * a.gate_stride + (a.head_gate ? h : h * a.Dv + d)));
+}
+// what the sink adds to a sum of weights exp2(score - m)
+__device__ __forceinline__ float window_sink(const WindowArgs& a, float m) { return a.sink ? exp2f(-m) : 0.0f; }
 
 // ---- general form: one wavefront per (token, query head) ---------------------------------------
 template <typename T>
@@ -78,13 +87,12 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WindowArgs a) {
                 if (c * 64 + lane < a.Dv) acc[c] += py * ld(vr + c * 64 + lane);
         }
     }
-    const float inv = 1.0f / l;
-    const T* gr = (const T*)a.gate + (int64_t)(t0 + t) * a.gate_stride + h * a.Dv;
+    const float inv = 1.0f / (l + window_sink(a, m));
     T* o = (T*)a.out + ((int64_t)(t0 + t) * a.H + h) * a.Dv;
 #pragma unroll
     for (int c = 0; c < 8; ++c) {
         const int d = c * 64 + lane;
-        if (d < a.Dv) st(o + d, acc[c] * inv * sigmoid_fast(ld(gr + d)));
+        if (d < a.Dv) st(o + d, acc[c] * inv * window_gate<T>(a, t0 + t, h, d));
     }
 }
 
@@ -228,8 +236,7 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowArgs a) {
         }
         const int h = g * per + h0 + x;
         if (a.splits == 1) {
-            const float gate = sigmoid_fast(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
-            st((T*)a.out + ((int64_t)b * a.H + h) * a.Dv + d, num / den * gate);
+            st((T*)a.out + ((int64_t)b * a.H + h) * a.Dv + d, num / (den + window_sink(a, mm)) * window_gate<T>(a, b, h, d));
         } else {
             float* w = a.ws + (((int64_t)b * a.H + h) * a.splits + split) * (a.Dv + 2);
             w[d] = num;
@@ -253,15 +260,14 @@ __global__ __launch_bounds__(256) void window_combine_kernel(WindowArgs a) {
     const float mm = fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3]));
     __syncthreads();
     const float e = __builtin_amdgcn_exp2f(m - mm);
-    const float inv = 1.0f / block_sum_f(l * e, part, 4);
+    const float inv = 1.0f / (block_sum_f(l * e, part, 4) + window_sink(a, mm));
     f[tid] = e * inv;
     __syncthreads();
     for (int d = tid; d < a.Dv; d += 256) {
         float num = 0.0f;
 #pragma unroll 8
         for (int s = 0; s < a.splits; ++s) num += w[s * row + d] * f[s];
-        const float gate = sigmoid_fast(ld((const T*)a.gate + b * a.gate_stride + h * a.Dv + d));
-        st((T*)a.out + bh * a.Dv + d, num * gate);
+        st((T*)a.out + bh * a.Dv + d, num * window_gate<T>(a, b, h, d));
     }
 }
 
@@ -491,8 +497,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
     }
     l += __shfl_xor(l, 32, 64);                            // the halves of a row hold disjoint keys
     if (!ok) return;
-    const float inv = 1.0f / l;
+    float inv = 1.0f / (l + window_sink(a, m));
     const bf16_t* gr = (const bf16_t*)a.gate + (int64_t)(tok0 + t) * a.gate_stride + h * a.Dv;
+    if (a.head_gate) inv *= window_gate<bf16_t>(a, tok0 + t, h, 0);
     bf16_t* orow = (bf16_t*)a.out + ((int64_t)(tok0 + t) * a.H + h) * a.Dv;
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
@@ -500,7 +507,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
         for (int c = 0; c < 4; ++c) {
             const int d = db * 32 + 8 * c + 4 * hl;
             if (a.vec) {
-                if (d < a.Dv) {
+                if (d >= a.Dv) continue;
+                if (a.head_gate) st4(orow + d, make_float4(o[db][4 * c] * inv, o[db][4 * c + 1] * inv, o[db][4 * c + 2] * inv, o[db][4 * c + 3] * inv));
+                else {
                     const float4 gt = ld4(gr + d);
                     st4(orow + d, make_float4(o[db][4 * c] * inv * sigmoid_fast(gt.x), o[db][4 * c + 1] * inv * sigmoid_fast(gt.y),
                                               o[db][4 * c + 2] * inv * sigmoid_fast(gt.z), o[db][4 * c + 3] * inv * sigmoid_fast(gt.w)));
@@ -508,7 +517,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
             } else {
 #pragma unroll
                 for (int x = 0; x < 4; ++x)
-                    if (d + x < a.Dv) st(orow + d + x, o[db][4 * c + x] * inv * sigmoid_fast(ld(gr + d + x)));
+                    if (d + x < a.Dv) st(orow + d + x, o[db][4 * c + x] * inv * (a.head_gate ? 1.0f : sigmoid_fast(ld(gr + d + x))));
             }
         }
     }
@@ -571,13 +580,13 @@ extern "C" int trimkv_window_decode_splits(int batch, int kv_heads, int capacity
 
 extern "C" int trimkv_window_decode(const void* q, const void* ring_k, const void* ring_v, const int32_t* slots, const int32_t* seen,
                                     const void* gate, int64_t gate_stride, void* out, int batch, int heads, int kv_heads, int dim, int vdim,
-                                    int dim_stride, int vdim_stride, int keep_first, int window, float scale, int splits, float* workspace,
+                                    int dim_stride, int vdim_stride, int keep_first, int window, float scale, int head_gate, int sink, int splits, float* workspace,
                                     int dtype, void* stream) {
     const char* fn = "trimkv_window_decode";
     WindowArgs a{};
     a.q = q; a.rk = ring_k; a.rv = ring_v; a.slots = slots; a.seen = seen; a.gate = gate; a.gate_stride = gate_stride; a.out = out;
     a.H = heads; a.G = kv_heads; a.D = dim; a.Dv = vdim; a.Dp = dim_stride; a.Dvp = vdim_stride; a.keep = keep_first; a.size = window;
-    a.scale_log2 = scale * 1.4426950408889634f; a.splits = splits; a.ws = workspace;
+    a.scale_log2 = scale * 1.4426950408889634f; a.splits = splits; a.ws = workspace; a.head_gate = head_gate; a.sink = sink;
     if (int rc = window_common(fn, a, batch, dtype)) return rc;
     if (splits < 1 || splits > 256 || (splits > 1 && !workspace)) return fail(TRIMKV_ERR_WORKSPACE, "%s: splits=%d needs a workspace", fn, splits);
     const int cap = keep_first + window;
@@ -599,12 +608,12 @@ extern "C" int trimkv_window_decode(const void* q, const void* ring_k, const voi
 extern "C" int trimkv_window_prefill(const void* q, const void* k, const void* v, const void* ring_k, const void* ring_v, const int32_t* cu,
                                      const int32_t* slots, const int32_t* seen, const void* gate, int64_t gate_stride, void* out, int batch, int max_len,
                                      int heads, int kv_heads, int dim, int vdim, int dim_stride, int vdim_stride, int keep_first, int window,
-                                     float scale, int dtype, void* stream) {
+                                     float scale, int head_gate, int sink, int dtype, void* stream) {
     const char* fn = "trimkv_window_prefill";
     WindowArgs a{};
     a.q = q; a.k = k; a.v = v; a.rk = ring_k; a.rv = ring_v; a.cu = cu; a.slots = slots; a.seen = seen; a.gate = gate; a.gate_stride = gate_stride; a.out = out;
     a.H = heads; a.G = kv_heads; a.D = dim; a.Dv = vdim; a.Dp = dim_stride; a.Dvp = vdim_stride; a.keep = keep_first; a.size = window;
-    a.scale_log2 = scale * 1.4426950408889634f; a.splits = 1;
+    a.scale_log2 = scale * 1.4426950408889634f; a.splits = 1; a.head_gate = head_gate; a.sink = sink;
     if (int rc = window_common(fn, a, batch, dtype)) return rc;
     if (!k || !v || !cu) return fail(TRIMKV_ERR_NULL, "%s: null pointer argument", fn);
     if (max_len <= 0 || (int64_t)batch * kv_heads > 65535) return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes max_len=%d batch*kv_heads=%lld", fn, max_len, (long long)batch * kv_heads);
@@ -612,7 +621,7 @@ extern "C" int trimkv_window_prefill(const void* q, const void* k, const void* v
     const int per = heads / kv_heads, big = dim_stride > vdim_stride ? dim_stride : vdim_stride;
     const bool aligned = !(((uintptr_t)k | (uintptr_t)v) & 15);
     if (dtype == TRIMKV_BF16 && big <= 256 && per <= 128 && aligned && scale > 0.0f) {
-        a.vec = vdim % 4 == 0 && gate_stride % 4 == 0 && !(((uintptr_t)gate | (uintptr_t)out) & 7);
+        a.vec = vdim % 4 == 0 && !((uintptr_t)out & 7) && (head_gate || (gate_stride % 4 == 0 && !((uintptr_t)gate & 7)));
         const int rc = big <= 64 ? launch_window_prefill<64>(a, batch, max_len, s) : big <= 128 ? launch_window_prefill<128>(a, batch, max_len, s)
                                                                                                : launch_window_prefill<256>(a, batch, max_len, s);
         if (rc) return fail(rc, "%s: hipFuncSetAttribute failed (%d)", fn, rc);

@@ -12,6 +12,7 @@ import torch
 # architecture name in config.json (``architecture``, or an entry of HF's ``architectures``) -> (module, class)
 MODELS = {
     "Fusitar": ("fusitar", "FusitarForCausalLM"),
+    "Siterax": ("siterax", "SiteraxForCausalLM"),
     "TrimKVQwen3ForCausalLM": ("qwen3", "TrimKVQwen3ForCausalLM"),
     "Qwen3ForCausalLM": ("qwen3", "TrimKVQwen3ForCausalLM"),
     "TrimKVLlamaForCausalLM": ("llama", "TrimKVLlamaForCausalLM"),
