@@ -634,6 +634,116 @@ HYBRID_SIZES = {
 }
 
 
+MFMA_PEAK, HBM_PEAK = 2500e12, 8e12
+
+
+def timed(fn, reps, warm=2):
+    """Seconds per call of ``fn(i)`` between two events."""
+    import torch
+    for i in range(warm):
+        fn(i)
+    torch.cuda.synchronize()
+    e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    e0.record()
+    for i in range(reps):
+        fn(i)
+    e1.record()
+    torch.cuda.synchronize()
+    return e0.elapsed_time(e1) * 1e-3 / reps
+
+
+def replayed(fn, reps):
+    """Seconds per call with ``reps`` calls recorded in one HIP graph: small launches are not timed at the host's pace."""
+    import torch
+    side = torch.cuda.Stream()
+    side.wait_stream(torch.cuda.current_stream())
+    with torch.cuda.stream(side):
+        for i in range(2):
+            fn(i)
+    torch.cuda.synchronize()
+    graph = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(graph, stream=side):
+        for i in range(reps):
+            fn(i)
+    return timed(lambda i: graph.replay(), 3, 1) / reps
+
+
+def roofline_entry(table, key, sec, flops=0.0, nbytes=0.0, note=None):
+    bound = max(flops / MFMA_PEAK, nbytes / HBM_PEAK)
+    table[key] = {"us": round(sec * 1e6, 1), "bound": "mfma" if flops / MFMA_PEAK >= nbytes / HBM_PEAK else "hbm", "frac_of_roofline": round(bound / sec, 3)}
+    if note:
+        table[key]["note"] = note
+
+
+def hybrid_shell(z, layers, vocab, rows, dev):
+    """The thin Qwen3 decoder at a hybrid decoder's width, head counts and attended rows, random bf16 weights."""
+    import torch
+    from trimkv_amd.qwen3 import TrimKVQwen3Config, TrimKVQwen3ForCausalLM
+    qcfg = TrimKVQwen3Config(vocab_size=vocab, hidden_size=z["W"], intermediate_size=3 * z["W"], num_hidden_layers=layers, num_attention_heads=z["Hq"],
+                             num_key_value_heads=z["Hkv"], head_dim=D, retention_gate="rg", retention_gate_bias_init=3.0, memory_size=rows, buffer_size=128)
+    torch.set_default_dtype(torch.bfloat16)
+    with torch.device(dev):
+        shell = TrimKVQwen3ForCausalLM(qcfg)
+    torch.set_default_dtype(torch.float32)
+    return shell.eval()
+
+
+def hybrid_throughput(r, label, model, shell, ids, B, M):
+    """Prompt and decode throughput of a hybrid decoder and the shell, in turn, into ``r``; returns the cache of the last batch
+    (B sequences of M tokens and a few more)."""
+    import torch
+    from trimkv_amd.graphed import GraphedDecoder
+    for b, s in ((1, 8192), (4, 2048)):
+        x = ids(b, s)
+
+        def prompt_new(i):
+            cache = model.new_cache(b)
+            model(x, past_key_values=cache, logits_to_keep=1)
+
+        both = []
+        for _ in range(2):
+            both.append((timed(prompt_new, 3), timed(lambda i: shell(x, logits_to_keep=1), 3)))
+        new_s, old_s = (min(t) for t in zip(*both))
+        r["prefill"][f"{b} x {s}"] = {f"{label}_tokens_per_s": round(b * s / new_s), "qwen3_shell_tokens_per_s": round(b * s / old_s),
+                                      f"{label}_ms": round(new_s * 1e3, 3), "qwen3_shell_ms": round(old_s * 1e3, 3)}
+    torch.cuda.empty_cache()
+    for b in sorted({1, B}):
+        cache, old = model.new_cache(b), None
+        x = ids(b, M)
+        step = max(1, 16384 // b)
+        for s0 in range(0, M, step):
+            model(x[:, s0:s0 + step], past_key_values=cache, logits_to_keep=1)
+            old = shell(x[:, s0:s0 + step], past_key_values=old, logits_to_keep=1).past_key_values
+        nxt = ids(b, 1)
+        n = 12
+        t_eager = timed(lambda i: model(nxt, past_key_values=cache, logits_to_keep=1), n)
+        o_eager = timed(lambda i: shell(nxt, past_key_values=old, logits_to_keep=1), n)
+        dec, odec = GraphedDecoder(model, cache, logits_to_keep=1), GraphedDecoder(shell, old, logits_to_keep=1)
+        t_graph = timed(lambda i: dec(input_ids=nxt), n, 3)
+        o_graph = timed(lambda i: odec(input_ids=nxt), n, 3)
+        t_graph, o_graph = min(t_graph, timed(lambda i: dec(input_ids=nxt), n)), min(o_graph, timed(lambda i: odec(input_ids=nxt), n))
+        dec.close()
+        odec.close()
+        r["decode"][f"batch {b}"] = {f"{label}_tokens_per_s": round(b / min(t_eager, t_graph)), "qwen3_shell_tokens_per_s": round(b / min(o_eager, o_graph)),
+                                     f"{label}_ms": {"eager": round(t_eager * 1e3, 3), "graph": round(t_graph * 1e3, 3)},
+                                     "qwen3_shell_ms": {"eager": round(o_eager * 1e3, 3), "graph": round(o_graph * 1e3, 3)}}
+        del old, dec, odec
+        if b != B:
+            del cache
+    torch.cuda.empty_cache()
+    return cache
+
+
+def hybrid_report(label, what, results):
+    first = next(iter(results.values()))
+    dec = first["decode"][max(first["decode"], key=lambda s: int(s.split()[1]))]
+    print(json.dumps({
+        "metric": f"decode tokens/s of the {label.capitalize()} decoder (4 layers, random weights) beside the thin Qwen3 decoder", "value": dec[f"{label}_tokens_per_s"], "unit": "tokens/s",
+        "n_gpus": 1, "steps": 12, "warmup": 2, "ms_per_step": min(dec[f"{label}_ms"].values()), "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
+        "data": "synthetic", "config": {"workload": f"4 layers ({what}), sizes per entry of `results`", "note": "secondary workload; the headline metric is the default run"},
+        "results": results}))
+
+
 def hybrid_main(args):
     """Secondary workload (--hybrid): the Fusitar decoder (two windowed-attention and two mLSTM layers, routed experts, random
     bf16 weights) beside the thin Qwen3 decoder at equal width, head counts, attended rows and weights read per token: prompt
@@ -643,38 +753,9 @@ def hybrid_main(args):
     import torch.nn.functional as F
     from trimkv_amd import _lib, hybrid_ops as ops, TrimKVCache, get_attention_interface
     from trimkv_amd.fusitar import FusitarConfig, FusitarForCausalLM
-    from trimkv_amd.graphed import GraphedDecoder
-    from trimkv_amd.qwen3 import TrimKVQwen3Config, TrimKVQwen3ForCausalLM
     dev = torch.device("cuda:0")
     torch.cuda.set_device(dev)
     gen = torch.Generator(device=dev).manual_seed(0)
-    MFMA, HBM = 2500e12, 8e12
-
-    def timed(fn, reps, warm=2):
-        for i in range(warm):
-            fn(i)
-        torch.cuda.synchronize()
-        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
-        e0.record()
-        for i in range(reps):
-            fn(i)
-        e1.record()
-        torch.cuda.synchronize()
-        return e0.elapsed_time(e1) * 1e-3 / reps
-
-    def replayed(fn, reps):
-        """Seconds per call with ``reps`` calls recorded in one HIP graph: small launches are not timed at the host's pace."""
-        side = torch.cuda.Stream()
-        side.wait_stream(torch.cuda.current_stream())
-        with torch.cuda.stream(side):
-            for i in range(2):
-                fn(i)
-        torch.cuda.synchronize()
-        graph = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(graph, stream=side):
-            for i in range(reps):
-                fn(i)
-        return timed(lambda i: graph.replay(), 3, 1) / reps
 
     results = {}
     for name in ([args.hybrid_size] if args.hybrid_size else list(HYBRID_SIZES)):
@@ -692,55 +773,12 @@ def hybrid_main(args):
         model.randomize()
         for i in (0, 2):
             model.model.layers[i].mix.f_bias.fill_(4.0)
-        qcfg = TrimKVQwen3Config(vocab_size=V, hidden_size=W, intermediate_size=3 * W, num_hidden_layers=L, num_attention_heads=z["Hq"], num_key_value_heads=z["Hkv"],
-                                 head_dim=D, retention_gate="rg", retention_gate_bias_init=3.0, memory_size=M, buffer_size=128)
-        torch.set_default_dtype(torch.bfloat16)
-        with torch.device(dev):
-            shell = TrimKVQwen3ForCausalLM(qcfg)
-        torch.set_default_dtype(torch.float32)
-        shell.eval()
+        shell = hybrid_shell(z, L, V, M, dev)
         ids = lambda b, s: torch.randint(0, V, (b, s), generator=gen, device=dev)
         r = results[name] = {"layers": L, "width": W, "prefill": {}, "decode": {}}
 
         with torch.no_grad():
-            for b, s in ((1, 8192), (4, 2048)):
-                x = ids(b, s)
-
-                def prompt_new(i):
-                    cache = model.new_cache(b)
-                    model(x, past_key_values=cache, logits_to_keep=1)
-
-                both = []
-                for _ in range(2):
-                    both.append((timed(prompt_new, 3), timed(lambda i: shell(x, logits_to_keep=1), 3)))
-                new_s, old_s = (min(t) for t in zip(*both))
-                r["prefill"][f"{b} x {s}"] = {"fusitar_tokens_per_s": round(b * s / new_s), "qwen3_shell_tokens_per_s": round(b * s / old_s),
-                                              "fusitar_ms": round(new_s * 1e3, 3), "qwen3_shell_ms": round(old_s * 1e3, 3)}
-            torch.cuda.empty_cache()
-            for b in sorted({1, B}):
-                cache, old = model.new_cache(b), None
-                x = ids(b, M)
-                step = max(1, 16384 // b)
-                for s0 in range(0, M, step):
-                    model(x[:, s0:s0 + step], past_key_values=cache, logits_to_keep=1)
-                    old = shell(x[:, s0:s0 + step], past_key_values=old, logits_to_keep=1).past_key_values
-                nxt = ids(b, 1)
-                n = 12
-                t_eager = timed(lambda i: model(nxt, past_key_values=cache, logits_to_keep=1), n)
-                o_eager = timed(lambda i: shell(nxt, past_key_values=old, logits_to_keep=1), n)
-                dec, odec = GraphedDecoder(model, cache, logits_to_keep=1), GraphedDecoder(shell, old, logits_to_keep=1)
-                t_graph = timed(lambda i: dec(input_ids=nxt), n, 3)
-                o_graph = timed(lambda i: odec(input_ids=nxt), n, 3)
-                t_graph, o_graph = min(t_graph, timed(lambda i: dec(input_ids=nxt), n)), min(o_graph, timed(lambda i: odec(input_ids=nxt), n))
-                dec.close()
-                odec.close()
-                r["decode"][f"batch {b}"] = {"fusitar_tokens_per_s": round(b / min(t_eager, t_graph)), "qwen3_shell_tokens_per_s": round(b / min(o_eager, o_graph)),
-                                             "fusitar_ms": {"eager": round(t_eager * 1e3, 3), "graph": round(t_graph * 1e3, 3)},
-                                             "qwen3_shell_ms": {"eager": round(o_eager * 1e3, 3), "graph": round(o_graph * 1e3, 3)}}
-                if b != B:
-                    del cache, old, dec, odec
-            del old, odec
-            torch.cuda.empty_cache()
+            cache = hybrid_throughput(r, "fusitar", model, shell, ids, B, M)
 
             # ---- kernel by kernel ----------------------------------------------------------------------
             T = 8192
@@ -750,12 +788,7 @@ def hybrid_main(args):
             big = torch.randn(T, xw, generator=gen, device=dev)
             bigh = big.to(torch.bfloat16)
 
-            def put(key, sec, flops=0.0, nbytes=0.0, note=None):
-                bound = max(flops / MFMA, nbytes / HBM)
-                k[key] = {"us": round(sec * 1e6, 1), "bound": "mfma" if flops / MFMA >= nbytes / HBM else "hbm", "frac_of_roofline": round(bound / sec, 3)}
-                if note:
-                    k[key]["note"] = note
-
+            put = lambda key, sec, **kw: roofline_entry(k, key, sec, **kw)
             pcache = model.new_cache(1)
             (slot,) = pcache.allocate(1)
             pb = pcache.batch([T], [slot])
@@ -772,7 +805,7 @@ def hybrid_main(args):
 
             def window_prefill(i):
                 _lib.check_hybrid(lib.trimkv_window_prefill(q.data_ptr(), kk.data_ptr(), vv.data_ptr(), ring["k"].data_ptr(), ring["v"].data_ptr(), pb.cu_dev.data_ptr(),
-                                                            pb.slots_dev.data_ptr(), pb.seen_dev.data_ptr(), gate, proj.stride(0), out.data_ptr(), 1, T, *shape, spec.scale, _lib.BF16, st), "window")
+                                                            pb.slots_dev.data_ptr(), pb.seen_dev.data_ptr(), gate, proj.stride(0), out.data_ptr(), 1, T, *shape, spec.scale, 0, 0, _lib.BF16, st), "window")
             seen_pairs = sum(min(t + 1, spec.window + min(spec.keep_first, max(0, t + 1 - spec.window))) for t in range(T))
             put("window_prefill", timed(window_prefill, 10), flops=4.0 * D * spec.heads * seen_pairs, note=f"{T} tokens")
             attn = get_attention_interface("trimkv_hip")
@@ -826,7 +859,7 @@ def hybrid_main(args):
             def window_decode(i):
                 rg = cache.layers_state[1 + 2 * (i % 2)]
                 _lib.check_hybrid(lib.trimkv_window_decode(qd.data_ptr(), rg["k"].data_ptr(), rg["v"].data_ptr(), db.slots_dev.data_ptr(), db.seen_dev.data_ptr(), aproj.data_ptr() + starts[3] * 2,
-                                                           aproj.stride(0), od.data_ptr(), B, *shape, spec.scale, splits, ws.data_ptr(), _lib.BF16, _lib.current_stream(dev)), "window")
+                                                           aproj.stride(0), od.data_ptr(), B, *shape, spec.scale, 0, 0, splits, ws.data_ptr(), _lib.BF16, _lib.current_stream(dev)), "window")
             put(f"window_decode (batch {B})", replayed(window_decode, 20), nbytes=2.0 * 2 * B * spec.kv_heads * spec.rows * D)
             oc = TrimKVCache()
             for l in range(2):
@@ -849,16 +882,148 @@ def hybrid_main(args):
             put(f"router product (decode, batch {B})", replayed(lambda i: ops.linear_f32(xd, moe_l.router), 20), nbytes=4.0 * B * W + 2.0 * z["E"] * W)
             put(f"shell: rmsnorm with residual (decode, batch {B})", replayed(lambda i: decoder_ops.rmsnorm(xdh, nw, 1e-6, xdh), 20), nbytes=B * W * 2.0 * 4)
             put(f"residual_norm (decode, batch {B})", replayed(lambda i: ops.residual_norm(xd, xdh, xdh, l_att[0].norm1, 1e-6), 20), nbytes=B * W * (2.0 + 4 + 4 + 2))
-        del model, shell, cache, dec
+        del model, shell, cache
         torch.cuda.empty_cache()
-    first = next(iter(results.values()))
-    dec = first["decode"][max(first["decode"], key=lambda s: int(s.split()[1]))]
-    ms = min(dec["fusitar_ms"].values())
-    print(json.dumps({
-        "metric": "decode tokens/s of the Fusitar decoder (4 layers, random weights) beside the thin Qwen3 decoder", "value": dec["fusitar_tokens_per_s"], "unit": "tokens/s",
-        "n_gpus": 1, "steps": 12, "warmup": 2, "ms_per_step": ms, "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-        "config": {"workload": "4 layers (mLSTM, windowed attention, twice), routed experts, sizes per entry of `results`", "note": "secondary workload; the headline metric is the default run"},
-        "results": results}))
+    hybrid_report("fusitar", "mLSTM, windowed attention, twice; routed experts", results)
+
+
+def siterax_main(args):
+    """Secondary workload (--hybrid --hybrid-model siterax): four layers of the Siterax decoder (windowed attention with rotary
+    positions and a sink, dense feed-forward, random bf16 weights) beside four of the thin Qwen3 decoder at equal width, head
+    counts, attended rows and feed-forward: throughput of both, and every kernel against its roofline next to the shell's."""
+    import torch
+    import torch.nn.functional as F
+    from trimkv_amd import _lib, decoder_ops, hybrid_ops as ops, TrimKVCache, get_attention_interface
+    from trimkv_amd.siterax import SiteraxConfig, SiteraxForCausalLM
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    gen = torch.Generator(device=dev).manual_seed(0)
+    rand = lambda *s: torch.randn(*s, generator=gen, device=dev)
+    half = lambda *s: rand(*s).to(torch.bfloat16)
+    results = {}
+    for name in ([args.hybrid_size] if args.hybrid_size else list(HYBRID_SIZES)):
+        z = HYBRID_SIZES[name]
+        W, Hq, Hkv, B, L, V, ff = z["W"], z["Hq"], z["Hkv"], args.batch or z["B"], 4, 1024, 3 * z["W"]
+        M = z["window"] + z["keep"]
+        layer = {"type": "attention", "mlp": {"kind": "dense", "ff": ff},
+                 "mixer": {"heads": Hq, "kv_heads": Hkv, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": M}, "rot": {"base": 1e6, "dims": D, "scaling": {"factor": 2.0}}}}
+        cfg = SiteraxConfig.from_dict({"vocab": V, "width": W, "norm": {"eps": 1e-6}, "residual_mult": 1.0, "logit_softcap": 30.0, "loop": {"start": 0, "stop": L, "times": 1}, "layers": [layer] * L})
+        with torch.device(dev):
+            model = SiteraxForCausalLM(cfg)
+        model.randomize()
+        shell = hybrid_shell(z, L, V, M, dev)
+        ids = lambda b, s: torch.randint(0, V, (b, s), generator=gen, device=dev)
+        r = results[name] = {"layers": L, "width": W, "window": M, "prefill": {}, "decode": {}}
+
+        class Mod:
+            training, num_key_value_groups = False, Hq // Hkv
+        attn = get_attention_interface("trimkv_hip")
+        with torch.no_grad():
+            cache = hybrid_throughput(r, "siterax", model, shell, ids, B, M)
+            T = 8192
+            k = r["kernels"] = {}
+            put = lambda key, sec, **kw: roofline_entry(k, key, sec, **kw)
+            lib = _lib.load_hybrid()
+            mixers = [l.mix for l in model.model.layers]
+            mix, l0 = mixers[0], model.model.layers[0]
+            spec, starts = mix.spec, mix.qkvg.starts("q", "k", "v", "g")
+            shape = (Hq, Hkv, D, D, D, D, 0, M)
+            heads = Hq + 2 * Hkv
+            code = _lib.BF16
+
+            def row_kernels(n, time):
+                """What is not a matrix product or attention, ``n`` tokens in a step; buffers of several layers in turn."""
+                x, y, stride = [rand(n, W) for _ in range(2)], [half(n, W) for _ in range(2)], ops.padded(W)
+                xh = torch.empty(n, stride, dtype=torch.bfloat16, device=dev)
+                tag = f"{n} tokens"
+                put(f"residual_norm with the next norm ({tag})", time(lambda i: ops.residual_norm(x[i % 2], xh, y[i % 2], l0.norm1b, 1e-6, None, 1.0, l0.norm2)), nbytes=n * W * (2.0 + 4 + 4 + 2))
+                nw = torch.ones(W, device=dev, dtype=torch.bfloat16)
+                put(f"shell: rmsnorm with residual ({tag})", time(lambda i: decoder_ops.rmsnorm(y[i % 2], nw, 1e-6, y[1 - i % 2])), nbytes=n * W * 2.0 * 4)
+                both = [half(n, 2 * ff) for _ in range(2)]
+                put(f"silu_gate ({tag})", time(lambda i: ops.silu_gate(both[i % 2], ff)), nbytes=n * ff * 2.0 * 3)
+                put(f"shell: silu_mul ({tag})", time(lambda i: decoder_ops.silu_mul(both[i % 2][:, :ff], both[i % 2][:, ff:])), nbytes=n * ff * 2.0 * 3)
+                toks = ids(1, n).reshape(-1)
+                stream = ops.embed_scaled(toks, model.model.embed, 1.0, stride, l0.norm1, 1e-6)
+                put(f"embedding with norm ({tag})", time(lambda i: ops.embed_scaled(toks, model.model.embed, 1.0, stride, l0.norm1, 1e-6)), nbytes=n * W * (2.0 + 4 + 2))
+                put(f"embedding added between passes ({tag})", time(lambda i: ops.embed_scaled(toks, model.model.embed, 1.0, stride, l0.norm1, 1e-6, add_to=stream)), nbytes=n * W * (2.0 + 4 + 4 + 2))
+                if n <= 64:
+                    logits = [half(n, 131072) for _ in range(2)]
+                    put(f"soft_cap ({n} x 131072)", time(lambda i: ops.soft_cap(logits[i % 2], 30.0)), nbytes=n * 131072 * 6.0)
+
+            row_kernels(T, lambda fn: timed(fn, 10))
+            row_kernels(B, lambda fn: replayed(fn, 20))
+
+            # prompt of T tokens
+            pcache = model.new_cache(1)
+            (slot,) = pcache.allocate(1)
+            pb = pcache.batch([T], [slot])
+            proj = half(T, mix.qkvg.weight.shape[0])
+            q, kk, vv = half(T, Hq, D), half(T, Hkv, D), half(T, Hkv, D)
+            out = torch.empty(T, Hq * D, dtype=torch.bfloat16, device=dev)
+            ring, st = pcache.layers_state[0], _lib.current_stream(dev)
+            table = ops.rotary_table(mix.rotation, mix.freq, pb)
+
+            def rotary_table(i):
+                pb.angles.clear()
+                ops.rotary_table(mix.rotation, mix.freq, pb)
+            put(f"rotary_table ({T} tokens, once per step)", timed(rotary_table, 10), nbytes=4.0 * T * D)
+            qkv = lambda p, t, dst, where, n, s: _lib.check_hybrid(lib.trimkv_qkv_heads(p.data_ptr(), p.stride(0), *starts[:3], mix.bias.data_ptr(), mix.q_norm.data_ptr(), mix.k_norm.data_ptr(), 1e-6,
+                                                                                      t.data_ptr(), D, Hq, Hkv, D, D, D, D, *(x.data_ptr() for x in dst), *where, n, code, s), "qkv_heads")
+            put(f"qkv_heads ({T} tokens)", timed(lambda i: qkv(proj, table, (q, kk, vv), (None, None, 0, 0), T, st), 10), nbytes=2.0 * 2 * T * heads * D + 4.0 * T * D)
+            cos = sin = half(1, T, D)
+            qw = torch.ones(D, device=dev, dtype=torch.bfloat16)
+            part = lambda p, n, at, cnt: p[:, at:at + cnt * D].unflatten(1, (cnt, D)).view(*n, cnt, D)
+            shell_qkv = lambda p, n, c: decoder_ops.qk_norm_rope(part(p, n, starts[0], Hq), part(p, n, starts[1], Hkv), qw, qw, c, c, 1e-6, part(p, n, starts[2], Hkv))
+            put(f"shell: qk_norm_rope ({T} tokens)", timed(lambda i: shell_qkv(proj, (1, T), cos), 10), nbytes=2.0 * 2 * T * heads * D + 2.0 * 2 * T * D)
+            gate = proj.data_ptr() + starts[3] * 2
+
+            def window_prefill(i):
+                _lib.check_hybrid(lib.trimkv_window_prefill(q.data_ptr(), kk.data_ptr(), vv.data_ptr(), ring["k"].data_ptr(), ring["v"].data_ptr(), pb.cu_dev.data_ptr(), pb.slots_dev.data_ptr(),
+                                                            pb.seen_dev.data_ptr(), gate, proj.stride(0), out.data_ptr(), 1, T, *shape, spec.scale, 1, 1, code, st), "window")
+            put(f"window_prefill ({T} tokens)", timed(window_prefill, 10), flops=4.0 * D * Hq * sum(min(t + 1, M) for t in range(T)))
+            oc = TrimKVCache()
+            K_, V_, _, _, kw = oc.update(kk.view(1, T, -1, D).transpose(1, 2), vv.view(1, T, -1, D).transpose(1, 2), torch.zeros(1, Hkv, T, device=dev), torch.arange(T, device=dev), 0)
+            q4 = q.view(1, T, -1, D).transpose(1, 2)
+            put(f"shell: prefill attention ({T} tokens, causal)", timed(lambda i: attn(Mod(), q4, K_, V_, None, scaling=D ** -0.5, flash_attn_kwargs=kw), 10), flops=4.0 * D * Hq * T * (T + 1) / 2)
+            put(f"ring_store ({T} tokens)", timed(lambda i: _lib.check_hybrid(lib.trimkv_ring_store(kk.data_ptr(), vv.data_ptr(), pb.cu_dev.data_ptr(), pb.slots_dev.data_ptr(), pb.seen_dev.data_ptr(),
+                                                                                                   ring["k"].data_ptr(), ring["v"].data_ptr(), 1, T, Hkv, D, D, 0, M, code, st), "store"), 10),
+                nbytes=2.0 * 2 * 2 * min(T, M) * Hkv * D)
+            xb = half(T, W)
+            put(f"vendor GEMM gate and up ({T} tokens)", timed(lambda i: F.linear(xb, model.model.layers[i % 4].mlp.gate_up.weight), 8), flops=2.0 * T * 2 * ff * W)
+            del oc, K_, V_, proj, q, kk, vv, out, pcache, ring, table, cos, sin, xb
+            torch.cuda.empty_cache()
+
+            # decode, batch B, windows full; layers alternate so that nothing stays in a cache
+            db = cache.batch([1] * B)
+            dproj, qd, od = half(B, mix.qkvg.weight.shape[0]), half(B, Hq, D), torch.empty(B, Hq * D, dtype=torch.bfloat16, device=dev)
+            splits = lib.trimkv_window_decode_splits(B, Hkv, spec.rows)
+            ws = torch.empty(B * Hq * splits * (D + 2), device=dev)
+
+            def window_decode(i):
+                rg = cache.layers_state[i % 4]
+                _lib.check_hybrid(lib.trimkv_window_decode(qd.data_ptr(), rg["k"].data_ptr(), rg["v"].data_ptr(), db.slots_dev.data_ptr(), db.seen_dev.data_ptr(), dproj.data_ptr() + starts[3] * 2,
+                                                           dproj.stride(0), od.data_ptr(), B, *shape, spec.scale, 1, 1, splits, ws.data_ptr(), code, _lib.current_stream(dev)), "window")
+            put(f"window_decode (batch {B})", replayed(window_decode, 20), nbytes=2.0 * 2 * B * Hkv * M * D)
+            dtable = ops.rotary_table(mix.rotation, mix.freq, db)
+            put(f"qkv_heads into the ring (batch {B})", replayed(lambda i: qkv(dproj, dtable, (qd, cache.layers_state[i % 4]["k"], cache.layers_state[i % 4]["v"]),
+                (db.slots_dev.data_ptr(), db.seen_dev.data_ptr(), 0, M), B, _lib.current_stream(dev)), 20), nbytes=2.0 * 2 * B * heads * D + 4.0 * B * D)
+            dcos = half(B, 1, D)
+            put(f"shell: qk_norm_rope (batch {B})", replayed(lambda i: shell_qkv(dproj, (B, 1), dcos), 20), nbytes=2.0 * 2 * B * heads * D + 4.0 * B * D)
+            oc = TrimKVCache()
+            for l in range(4):
+                kd = half(B, Hkv, M, D)
+                oc.update(kd, kd, torch.zeros(B, Hkv, M, device=dev), torch.arange(M, device=dev), l)
+            del kd
+            q4 = qd.view(B, Hq, 1, D)
+            views = [(oc.key_cache[l], oc.value_cache[l], {"seg_len": oc._slabs[l].seg_len, "max_len": M, "seg_cap": oc._slabs[l].cap}) for l in range(4)]
+            put(f"shell: decode attention (batch {B})", replayed(lambda i: attn(Mod(), q4, views[i % 4][0], views[i % 4][1], None, scaling=D ** -0.5, flash_attn_kwargs=views[i % 4][2]), 20),
+                nbytes=2.0 * 2 * B * Hkv * M * D)
+            xb = half(B, W)
+            put(f"vendor GEMM gate and up (batch {B})", replayed(lambda i: F.linear(xb, model.model.layers[i % 4].mlp.gate_up.weight), 20), nbytes=2.0 * 2 * ff * W)
+            del oc, views
+        del model, shell, cache
+        torch.cuda.empty_cache()
+    hybrid_report("siterax", "windowed attention, dense feed-forward", results)
 
 
 def main():
@@ -901,8 +1066,9 @@ def main():
                     help="secondary workload: chunked prompt processing at config 5's shape (4096-token chunks); "
                          "with it --steps/--warmup count chunks (defaults 6/2)")
     ap.add_argument("--hybrid", action="store_true",
-                    help="secondary workload: prompt and decode throughput of the Fusitar decoder beside the thin Qwen3 decoder at equal size, "
+                    help="secondary workload: prompt and decode throughput of the Fusitar (--hybrid-model siterax: the Siterax) decoder beside the thin Qwen3 decoder at equal size, "
                          "and its kernels against their rooflines")
+    ap.add_argument("--hybrid-model", choices=("fusitar", "siterax"), default="fusitar", help="--hybrid only: which decoder")
     ap.add_argument("--hybrid-size", choices=sorted(HYBRID_SIZES), help="--hybrid only: one of the sizes (default: all)")
     args = ap.parse_args()
     if args.event_every < 0:
@@ -917,7 +1083,7 @@ def main():
             args.steps, args.warmup = 6, 2
         return prefill_main(args)
     if args.hybrid:
-        return hybrid_main(args)
+        return siterax_main(args) if args.hybrid_model == "siterax" else hybrid_main(args)
     if args.shell:
         if args.steps == 1024 and args.warmup == 128:
             args.steps, args.warmup = 12, 3

@@ -71,7 +71,8 @@ int trimkv_silu_gate(const void* gate, const void* up, int64_t stride, void* out
 int trimkv_soft_cap(const void* x, float* out, int64_t count, float cap, int dtype, void* stream);
 
 /* Window rings [slot][kv_heads][keep_first + window][dim_stride]: position p < keep_first owns row p, a later one row
- * keep_first + (p - keep_first) % window.  Stores those tokens of a portion that no later token of it overwrites. */
+ * keep_first + (p - keep_first) % window.  Stores those tokens of a portion that no later token of it overwrites.
+ * Padded sizes are multiples of 8, pointers 16-byte aligned. */
 int trimkv_ring_store(const void* k, const void* v, const int32_t* cu, const int32_t* slots, const int32_t* seen, void* ring_k, void* ring_v,
                       int batch, int max_len, int kv_heads, int dim_stride, int vdim_stride, int keep_first, int window, int dtype, void* stream);
 

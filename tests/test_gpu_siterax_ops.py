@@ -173,6 +173,8 @@ LAYERS = {
     "no_turn": (4, 2, 32, 40, 33, 0, 0.2),
     "group_of_eight": (8, 1, 128, 128, 70, 128, 0.09),
     "group_of_twelve": (12, 1, 40, 8, 33, 16, 0.2),
+    "between_tiles": (6, 2, 96, 72, 50, 64, 0.12),
+    "between_tiles_values": (4, 1, 72, 88, 90, 32, 0.15),
     "wide": (4, 2, 200, 96, 64, 48, 0.07),
     "long_window": (4, 1, 64, 64, 300, 64, 0.15),
     "widest": (2, 1, 320, 272, 40, 320, 0.05),

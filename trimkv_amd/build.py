@@ -27,6 +27,8 @@ HIPCC_FLAGS = [
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     "-Wno-unused-value",
 ]
+# maxima of scores: without this every operand of fmaxf is first run through v_max_f32 to quiet a NaN that cannot be there
+EXTRA_FLAGS = {"window_attn.hip": ["-fno-honor-nans"]}
 
 
 def _run(cmd):
@@ -58,7 +60,7 @@ def build(verbose: bool = True, only_changed: bool = False, libraries=tuple(LIBR
         srcs = [s for s in srcs if _stale(s, obj_of(s))]
 
     def compile_one(src):
-        return _run([hipcc] + HIPCC_FLAGS + ["-c", os.path.join(CSRC, src), "-o", obj_of(src)])
+        return _run([hipcc] + HIPCC_FLAGS + EXTRA_FLAGS.get(src, []) + ["-c", os.path.join(CSRC, src), "-o", obj_of(src)])
 
     if srcs:
         with ThreadPoolExecutor(max_workers=min(os.cpu_count() or 4, 8, len(srcs))) as ex:

@@ -536,24 +536,19 @@ __global__ __launch_bounds__(256) void soft_cap_kernel(const T* x, float* out, i
 }
 
 // ---- a prompt's surviving rows into the ring -----------------------------------------------------
-template <typename T>
-__global__ __launch_bounds__(256) void ring_store_kernel(const T* k, const T* v, const int32_t* cu, const int32_t* slots, const int32_t* seen,
-                                                         T* rk, T* rv, int G, int Dp, int Dvp, int keep, int size) {
+// Rows are multiples of 16 bytes: kc pieces of 16 for a token's keys of one head, vc for its values.
+__global__ __launch_bounds__(256) void ring_store_kernel(const uint4* k, const uint4* v, const int32_t* cu, const int32_t* slots, const int32_t* seen,
+                                                         uint4* rk, uint4* rv, int G, int kc, int vc, int keep, int size) {
     const int b = blockIdx.y, slot = slots[b], t0 = cu[b], len = cu[b + 1] - t0, past = seen[2 * slot];
     const int i = blockIdx.x;                          // token of the portion
     if (i >= len) return;
     const int pos = past + i;
     if (pos >= keep && pos < past + len - size) return;     // a later token takes its slot
     const int cap = keep + size, r = ring_slot(pos, keep, size);
-    const T* ks = k + (int64_t)(t0 + i) * G * Dp;
-    const T* vs = v + (int64_t)(t0 + i) * G * Dvp;
-    for (int e = threadIdx.x; e < G * Dp; e += 256) {
-        const int g = e / Dp, d = e - g * Dp;
-        rk[(((int64_t)slot * G + g) * cap + r) * Dp + d] = ks[e];
-    }
-    for (int e = threadIdx.x; e < G * Dvp; e += 256) {
-        const int g = e / Dvp, d = e - g * Dvp;
-        rv[(((int64_t)slot * G + g) * cap + r) * Dvp + d] = vs[e];
+    for (int e = threadIdx.x; e < G * (kc + vc); e += 256) {
+        const bool key = e < G * kc;
+        const int n = key ? kc : vc, at = key ? e : e - G * kc, g = at / n;
+        (key ? rk : rv)[(((int64_t)slot * G + g) * cap + r) * n + (at - g * n)] = (key ? k : v)[(int64_t)(t0 + i) * G * n + at];
     }
 }
 
@@ -788,8 +783,11 @@ extern "C" int trimkv_ring_store(const void* k, const void* v, const int32_t* cu
     HY_CHECK_DTYPE(fn, dtype);
     if (batch <= 0 || batch > 65535 || max_len <= 0 || kv_heads <= 0 || dim_stride <= 0 || vdim_stride <= 0 || keep_first < 0 || window <= 0)
         return fail(TRIMKV_ERR_SHAPE, "%s: bad sizes batch=%d max_len=%d kv_heads=%d keep=%d window=%d", fn, batch, max_len, kv_heads, keep_first, window);
-    HY_BY_DTYPE(dtype, T, hipLaunchKernelGGL((ring_store_kernel<T>), dim3(max_len, batch), dim3(256), 0, (hipStream_t)stream,
-                                             (const T*)k, (const T*)v, cu, slots, seen, (T*)ring_k, (T*)ring_v, kv_heads, dim_stride, vdim_stride, keep_first, window));
+    const int per = dtype == TRIMKV_BF16 ? 8 : 4;
+    if (dim_stride % 8 || vdim_stride % 8 || (((uintptr_t)k | (uintptr_t)v | (uintptr_t)ring_k | (uintptr_t)ring_v) & 15))
+        return fail(TRIMKV_ERR_SHAPE, "%s: padded sizes must be multiples of 8 and pointers 16-byte aligned", fn);
+    hipLaunchKernelGGL(ring_store_kernel, dim3(max_len, batch), dim3(256), 0, (hipStream_t)stream, (const uint4*)k, (const uint4*)v, cu, slots, seen,
+                       (uint4*)ring_k, (uint4*)ring_v, kv_heads, dim_stride / per, vdim_stride / per, keep_first, window);
     return launch_status(fn);
 }
 

@@ -286,10 +286,11 @@ struct WindowTile {
     static __device__ __forceinline__ int vswz(int r) { return D == 64 ? 4 * ((r >> 1) & 1) : 4 * (r & 3); }   // in 16-byte pieces
 };
 
-template <int D>
+// Tiles are laid out for D features; products stop at USED of them.
+template <int D, int USED>
 __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(WindowArgs a) {
     using W = WindowTile<D>;
-    constexpr int KS = D / 16, DB = D / 32;
+    constexpr int KS = USED / 16, DB = USED / 32;
     extern __shared__ __attribute__((aligned(16))) char wa_lds[];
     HY_LDS char* const lds3 = (HY_LDS char*)wa_lds;
     const uint32_t lds0 = (uint32_t)(uintptr_t)lds3;
@@ -399,6 +400,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
         const int off = (n & 1) * 2 * W::TILE;
         // operands are requested AHEAD steps before the MFMA that takes them; the fences keep the compiler from moving them back
         constexpr int AHEAD = 3;
+        __builtin_amdgcn_s_setprio(1);                     // the wavefront that can feed the matrix cores goes first
         hy_f32x16 s[2];
 #pragma unroll
         for (int v = 0; v < 16; ++v) s[0][v] = s[1][v] = 0.0f;
@@ -416,6 +418,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
         hy_bf16x8 vf[4 * DB];
 #pragma unroll
         for (int x = 0; x < AHEAD; ++x) vf[x] = v_frag(off, x / DB, x % DB);
+        __builtin_amdgcn_s_setprio(0);
         const bool whole = !ring && k0 + 63 <= tw0 && (k0 > tw1 - a.size || past + k0 + 63 < a.keep);
         if (!whole) {
             asm volatile("" :::);                          // keeps this a branch
@@ -477,6 +480,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
         };
 #pragma unroll
         for (int x = 0; x < 4; ++x) weigh(0, x);
+        __builtin_amdgcn_s_setprio(1);
 #pragma unroll
         for (int st_ = 0; st_ < 4; ++st_) {
 #pragma unroll
@@ -494,6 +498,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
                 __builtin_amdgcn_sched_barrier(0);
             }
         }
+        __builtin_amdgcn_s_setprio(0);
     }
     l += __shfl_xor(l, 32, 64);                            // the halves of a row hold disjoint keys
     if (!ok) return;
@@ -523,19 +528,19 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void window_prefill_kernel(W
     }
 }
 
-template <int D>
+template <int D, int USED = D>
 static int launch_window_prefill(const WindowArgs& a, int batch, int max_len, hipStream_t s) {
     constexpr int LDS = 4 * WindowTile<D>::TILE;
     static bool opted_in[64] = {};
     int dev = 0;
     if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) dev = -1;
     if (dev < 0 || !opted_in[dev]) {
-        hipError_t e = hipFuncSetAttribute((const void*)window_prefill_kernel<D>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
+        hipError_t e = hipFuncSetAttribute((const void*)window_prefill_kernel<D, USED>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
         if (e != hipSuccess) return (int)e;
         if (dev >= 0) opted_in[dev] = true;
     }
     const int bt = 128 / (a.H / a.G);
-    hipLaunchKernelGGL((window_prefill_kernel<D>), dim3((max_len + bt - 1) / bt, batch * a.G), dim3(256), LDS, s, a);
+    hipLaunchKernelGGL((window_prefill_kernel<D, USED>), dim3((max_len + bt - 1) / bt, batch * a.G), dim3(256), LDS, s, a);
     return 0;
 }
 
@@ -622,7 +627,7 @@ extern "C" int trimkv_window_prefill(const void* q, const void* k, const void* v
     const bool aligned = !(((uintptr_t)k | (uintptr_t)v) & 15);
     if (dtype == TRIMKV_BF16 && big <= 256 && per <= 128 && aligned && scale > 0.0f) {
         a.vec = vdim % 4 == 0 && !((uintptr_t)out & 7) && (head_gate || (gate_stride % 4 == 0 && !((uintptr_t)gate & 7)));
-        const int rc = big <= 64 ? launch_window_prefill<64>(a, batch, max_len, s) : big <= 128 ? launch_window_prefill<128>(a, batch, max_len, s)
+        const int rc = big <= 64 ? launch_window_prefill<64>(a, batch, max_len, s) : big <= 96 ? launch_window_prefill<128, 96>(a, batch, max_len, s) : big <= 128 ? launch_window_prefill<128>(a, batch, max_len, s)
                                                                                                : launch_window_prefill<256>(a, batch, max_len, s);
         if (rc) return fail(rc, "%s: hipFuncSetAttribute failed (%d)", fn, rc);
         return launch_status(fn);
